@@ -1,4 +1,5 @@
-"""Plain restatement of a layered decoder (attention with pooled blocks, gated delta rule, retention) in numpy.
+"""Plain restatement of layered decoders in numpy: Suripel (attention with pooled blocks, gated delta rule, retention) and
+Lesarax (attention with sinks whose values are its keys, latent attention, mixture of experts, looped layers).
 
 Test infrastructure only: one function per mechanism, whole sequences at once or token by token from the
 equations, in float64, sharing nothing with the product path. A model is (config, weights): the dictionary of
@@ -76,6 +77,10 @@ def layer_norm(x, w, eps):
 
 def over_rms(x, eps):
     return x / np.sqrt((x * x).mean(-1, keepdims=True) + eps)
+
+
+def rms_norm(x, w, eps):
+    return over_rms(x, eps) * w
 
 
 def unit(x):
@@ -203,8 +208,106 @@ def feed_forward(cfg, w, p, h):
     return polynorm(h @ w[p + "up"].T, w[p + "act"], cfg["norm"]["eps"]) @ w[p + "down"].T
 
 
+# ---------------------------------------------------------------------------------------------- Lesarax
+def sink_attention(q, k, v, scale, sinks, size=None):
+    """q [T][H][d], k [T][G][d], v [T][G][dv] -> [T][H][dv]: causal, over the last `size` tokens (None: all of them), with
+    exp(sink of the head) as one more term of the softmax's denominator."""
+    T, H = q.shape[:2]
+    rep = H // k.shape[1]
+    out = np.zeros((T, H, v.shape[2]), dtype=F)
+    for i in range(T):
+        lo = 0 if size is None else max(0, i - size + 1)
+        for h in range(H):
+            s = k[lo:i + 1, h // rep] @ q[i, h] * scale
+            top = max(s.max(), sinks[h])
+            p = np.exp(s - top)
+            out[i, h] = p @ v[lo:i + 1, h // rep] / (p.sum() + np.exp(sinks[h] - top))
+    return out
+
+
+def rotate_rows(x, rot):
+    """x [T][heads][dim], row t at position t."""
+    return np.stack([rotate_half(x[t], t, rot["dims"], rot["base"]) for t in range(x.shape[0])])
+
+
+def mixer_tied_attention(cfg, w, p, mx, h):
+    """Rotary attention with sinks; the values are the keys before their rotation."""
+    T, H, G, d = h.shape[0], mx["heads"], mx["kv_heads"], mx["dim"]
+    q = (h @ w[p + "q"].T).reshape(T, H, d)
+    k = (h @ w[p + "k"].T).reshape(T, G, d)
+    o = sink_attention(rotate_rows(q, mx["rot"]), rotate_rows(k, mx["rot"]), k, mx["scale"], w[p + "sink"])
+    return o.reshape(T, H * d) @ w[p + "o"].T
+
+
+def mixer_latent_attention(cfg, w, p, mx, h):
+    """Queries from a normed latent, keys and values from another one, one rotated key part for all heads, sinks, a window
+    and a gate per head."""
+    T, H, d, r, dv = h.shape[0], mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"]
+    eps, rank = cfg["norm"]["eps"], mx["kv_rank"]
+    q = (rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], eps) @ w[p + "uq"].T).reshape(T, H, d + r)
+    ckv = h @ w[p + "dkv"].T
+    c = rms_norm(ckv[:, :rank], w[p + "dkv.norm"], eps)
+    k_rot = rotate_rows(ckv[:, None, rank:], mx["rot"])
+    q = np.concatenate([q[..., :d], rotate_rows(q[..., d:], mx["rot"])], -1)
+    k = np.concatenate([(c @ w[p + "uk"].T).reshape(T, H, d), np.repeat(k_rot, H, 1)], -1)
+    v = (c @ w[p + "uv"].T).reshape(T, H, dv)
+    o = sink_attention(q, k, v, mx["scale"], w[p + "sink"], mx["mask"]["size"])
+    o = o * sigmoid(h @ w[p + "g"].T)[..., None]
+    return o.reshape(T, H * dv) @ w[p + "o"].T
+
+
+def clamped_expert(h, gate, up, down, limit):
+    g = np.minimum(gate @ h, limit)
+    u = np.clip(up @ h, -limit, limit)
+    return down @ (g * sigmoid(1.702 * g) * (u + 1))
+
+
+def route(logits, top):
+    """(indices of the `top` largest, softmax over them)"""
+    pick = np.argsort(-logits, kind="stable")[:top]
+    e = np.exp(logits[pick] - logits[pick].max())
+    return pick, e / e.sum()
+
+
+def mixture_of_experts(w, p, mlp, h):
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        for e, a in zip(*route(w[p + "router"] @ h[t], mlp["router"]["top"])):
+            q = p + f"e{e}."
+            out[t] += a * clamped_expert(h[t], w[q + "gate"], w[q + "up"], w[q + "down"], mlp["expert"]["limit"])
+    return out
+
+
+def layer_runs(cfg):
+    """[(layer, whether it is the first one of a pass through the looped part)] in the order they run."""
+    lp = cfg["loop"]
+    runs = [(i, False) for i in range(lp["start"])]
+    for _ in range(lp["times"]):
+        runs += [(i, i == lp["start"]) for i in range(lp["start"], lp["stop"])]
+    return runs + [(i, False) for i in range(lp["stop"], len(cfg["layers"]))]
+
+
+def lesarax_forward(cfg, w, tokens, layers_out=None):
+    eps, m = cfg["norm"]["eps"], cfg["residual_mult"]
+    x0 = np.array(w["embed"][np.asarray(tokens)], dtype=F)
+    x = x0
+    for i, pass_starts in layer_runs(cfg):
+        layer, p = cfg["layers"][i], f"l{i}."
+        if pass_starts:
+            x = np.concatenate([x, x0], -1) @ w["loop.in"].T
+        mixer = {"attention": mixer_tied_attention, "latent_attention": mixer_latent_attention}[layer["type"]]
+        x = x + m * mixer(cfg, w, p + "mix.", layer["mixer"], rms_norm(x, w[p + "norm1"], eps))
+        if layer.get("mlp") is not None:
+            x = x + m * mixture_of_experts(w, p + "mlp.", layer["mlp"], rms_norm(x, w[p + "norm2"], eps))
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return rms_norm(x, w["final.norm"], eps) @ w["embed"].T
+
+
 def forward(cfg, w, tokens, layers_out=None):
     """Logits [T][vocab] of a whole sequence; appends the residual stream after every layer to layers_out."""
+    if cfg["architecture"] == "Lesarax":
+        return lesarax_forward(cfg, w, tokens, layers_out)
     eps = cfg["norm"]["eps"]
     x = np.array(w["embed"][np.asarray(tokens)], dtype=F)
     kv = {}
