@@ -94,6 +94,8 @@ ABI = {
     "w4a32_decoder_step": (_ci, [_vp, _vp, _vp, _vp, _vp, _vp]),
     # include/w4a32_layered.h
     "w4a32_layered_check": (_ci, [_vp]),
+    "w4a32_layered_head_rows": (_ci, [_ci, _ci]),
+    "w4a32_layered_runs": (_ci, [_vp]),
     "w4a32_layered_state_bytes": (_sz, [_vp]),
     "w4a32_layered_workspace_bytes": (_sz, [_vp]),
     "w4a32_layered_position_offset": (_sz, [_vp]),
@@ -107,6 +109,8 @@ ABI = {
     "w4a32_op_layernorm_conv": (_ci, [_vp, _vp, _ci, _vp, _vp, ctypes.c_float, _vp, _vp, _ci, _ci, _ci, _ci, _vp, _ci,
                                       _vp]),
     "w4a32_op_short_conv": (_ci, [_vp, _ci, _vp, _ci, _vp, _vp] + [_ci] * 6 + [_vp]),
+    "w4a32_op_experts_scratch_bytes": (_sz, [_ci, _ci, _ci, _ci, _ci]),
+    "w4a32_op_experts": (_ci, [_ci, _vp, _vp, _ci, _vp, _vp, _ci, _ci, _ci, _ci, _ci, ctypes.c_float, _vp, _vp, _vp]),
     "w4a32_op_polynorm": (_ci, [_vp, _ci, _ci, _ci, _ci, _vp, ctypes.c_float, _vp]),
 }
 
@@ -141,34 +145,40 @@ class DecoderWeights(ctypes.Structure):
 
 
 LAYERED_BF16, LAYERED_F32 = 1, 2
-MIXERS = {"attention": 1, "delta": 2, "retention": 3}
+MIXERS = {"attention": 1, "delta": 2, "retention": 3, "rotary": 4, "latent": 5}
+NORM_LAYER, NORM_RMS = 0, 1
 
 
 class LayerConfig(ctypes.Structure):
     """w4a32_layer_config"""
     _fields_ = [(n, ctypes.c_int) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "conv_taps")] + \
                [("scale", ctypes.c_float)] + [(n, ctypes.c_int) for n in ("window", "pool", "kv_from", "rot_dims")] + \
-               [("rot_base", ctypes.c_float), ("ff", ctypes.c_int)]
+               [("rot_base", ctypes.c_double)] + \
+               [(n, ctypes.c_int) for n in ("ff", "tied_values", "q_rank", "kv_rank", "rot_part", "head_gate", "experts",
+                                            "top")] + \
+               [("expert_limit", ctypes.c_float)]
 
 
 class LayeredConfig(ctypes.Structure):
     """w4a32_layered_config"""
     _fields_ = [(n, ctypes.c_int) for n in ("hidden", "vocab", "n_layers", "canon_taps")] + \
                [("norm_eps", ctypes.c_float)] + [(n, ctypes.c_int) for n in ("dtype", "max_seq", "max_batch_tokens")] + \
-               [("layers", ctypes.POINTER(LayerConfig))]
+               [("layers", ctypes.POINTER(LayerConfig)), ("norm", ctypes.c_int), ("residual_mult", ctypes.c_float)] + \
+               [(n, ctypes.c_int) for n in ("loop_start", "loop_stop", "loop_times")]
 
 
 class LayeredLayer(ctypes.Structure):
     """w4a32_layered_layer"""
     _fields_ = [(n, ctypes.c_void_p) for n in ("norm1", "norm2", "canon1", "canon2", "in_proj", "conv", "out_proj",
                                                "a_log", "dt_bias", "head_norm", "decay", "log_decay", "up", "down",
-                                               "act")]
+                                               "act", "sinks", "q_norm", "kv_norm", "q_up", "k_up", "v_up", "router",
+                                               "gate_up", "experts_down")]
 
 
 class LayeredWeights(ctypes.Structure):
     """w4a32_layered_weights"""
     _fields_ = [("embedding", ctypes.c_void_p), ("final_norm", ctypes.c_void_p), ("head", ctypes.c_void_p),
-                ("layers", ctypes.POINTER(LayeredLayer))]
+                ("layers", ctypes.POINTER(LayeredLayer)), ("loop_in", ctypes.c_void_p)]
 
 
 class W4A32Error(RuntimeError):
@@ -856,23 +866,73 @@ def op_polynorm(z, F, act, eps):
     return z
 
 
+def pack_operand_blocks(w, heads, rows):
+    """w [heads * n][K] -> the layout of k_up / v_up: `rows` rows per head (zeros behind the n true ones), columns padded to
+    64, in blocks [32 rows][8 columns]."""
+    import torch
+
+    K, n = _pad64(w.shape[1]), w.shape[0] // heads
+    full = torch.zeros((heads, rows, K), dtype=w.dtype, device=w.device)
+    full[:, :n, :w.shape[1]] = w.view(heads, n, -1)
+    return full.view(heads * rows // 32, 32, K // 8, 8).permute(0, 2, 1, 3).contiguous()
+
+
+def pack_gate_up(gate, up):
+    """gate, up [E][ff][K] -> [E][2 pad(ff)][pad(K)] in groups of 64 rows: 32 of gate, the same 32 of up."""
+    import torch
+
+    E, ff, K = gate.shape
+    out = torch.zeros((E, _pad64(ff) // 32, 2, 32, _pad64(K)), dtype=gate.dtype, device=gate.device)
+    for i, t in enumerate((gate, up)):
+        pad = torch.zeros((E, _pad64(ff), _pad64(K)), dtype=gate.dtype, device=gate.device)
+        pad[:, :ff, :K] = t
+        out[:, :, i] = pad.view(E, -1, 32, _pad64(K))
+    return out.view(E, 2 * _pad64(ff), _pad64(K))
+
+
+def op_experts(h, logits, gate_up, down, hidden, top, ff, limit):
+    """h [M][pad(hidden)] (bf16 or f32), logits [M][E], packed weights -> weighted rows [top][M][pad(hidden)] f32."""
+    import torch
+
+    M, E = logits.shape
+    dtype = LAYERED_BF16 if h.dtype == torch.bfloat16 else LAYERED_F32
+    parts = torch.empty((top, M, h.shape[1]), dtype=torch.float32, device="cuda")
+    scratch = _dev_empty(int(lib().w4a32_op_experts_scratch_bytes(dtype, M, E, top, ff)))
+    _check(lib().w4a32_op_experts(dtype, _ptr(h), _ptr(logits), E, _ptr(gate_up), _ptr(down), M, hidden, E, top, ff, limit,
+                                  _ptr(parts), _ptr(scratch), _stream()), "w4a32_op_experts")
+    return parts
+
+
 class LayeredDecoder:
     """Plumbing around the layered decoder runner: packs a model given as the dictionary of its config.json and a
     dictionary of cuda tensors under its parameter names, owns workspace and sequence states. The C++ classes in
     host/mllm/Models do the same from files."""
 
     def __init__(self, config, weights, dtype="bfloat16", max_seq=1024, max_batch_tokens=512):
-        import math
-
         import torch
 
         self.dtype = torch.bfloat16 if dtype == "bfloat16" else torch.float32
         self._keep = []
-        W, vocab, taps = config["width"], config["vocab"], config["canon"]["taps"]
         layers = config["layers"]
         self.layer_cfg = (LayerConfig * len(layers))()
         self.layer_w = (LayeredLayer * len(layers))()
-        for i, layer in enumerate(layers):
+        self.cfg = LayeredConfig(config["width"], config["vocab"], len(layers), 0, config["norm"]["eps"],
+                                 LAYERED_BF16 if dtype == "bfloat16" else LAYERED_F32, max_seq, max_batch_tokens,
+                                 self.layer_cfg)
+        {"Suripel": self._suripel, "Lesarax": self._lesarax}[config.get("architecture", "Suripel")](config, weights)
+        _check(lib().w4a32_layered_check(ctypes.byref(self.cfg)), "w4a32_layered_check")
+        self.ws = _dev_empty(int(lib().w4a32_layered_workspace_bytes(ctypes.byref(self.cfg))))
+        _check(lib().w4a32_layered_init_workspace(ctypes.byref(self.cfg), _ptr(self.ws), _stream()),
+               "w4a32_layered_init_workspace")
+        self.token = torch.zeros((1,), dtype=torch.int64, device="cuda")
+
+    def _suripel(self, config, weights):
+        import math
+
+        import torch
+
+        self.cfg.canon_taps = config["canon"]["taps"]
+        for i, layer in enumerate(config["layers"]):
             m, t, c, lw = layer["mixer"], layer["type"], self.layer_cfg[i], self.layer_w[i]
             p, mp = f"l{i}.", f"l{i}.mix."
             heads, dim, vdim = m["heads"], m["dim"], m["vdim"]
@@ -905,14 +965,48 @@ class LayeredDecoder:
                 lw.act = self._vector(weights[p + "mlp.act"])
         self.weights = LayeredWeights(self._matrix([weights["embed"]], False), self._vector(weights["final.norm"]),
                                       self._matrix([weights["head"]], False), self.layer_w)
-        self.cfg = LayeredConfig(W, vocab, len(layers), taps, config["norm"]["eps"],
-                                 LAYERED_BF16 if dtype == "bfloat16" else LAYERED_F32, max_seq, max_batch_tokens,
-                                 self.layer_cfg)
-        _check(lib().w4a32_layered_check(ctypes.byref(self.cfg)), "w4a32_layered_check")
-        self.ws = _dev_empty(int(lib().w4a32_layered_workspace_bytes(ctypes.byref(self.cfg))))
-        _check(lib().w4a32_layered_init_workspace(ctypes.byref(self.cfg), _ptr(self.ws), _stream()),
-               "w4a32_layered_init_workspace")
-        self.token = torch.zeros((1,), dtype=torch.int64, device="cuda")
+
+    def _lesarax(self, config, weights):
+        import torch
+
+        loop = config["loop"]
+        self.cfg.norm, self.cfg.residual_mult = NORM_RMS, config["residual_mult"]
+        self.cfg.loop_start, self.cfg.loop_stop, self.cfg.loop_times = loop["start"], loop["stop"], loop["times"]
+        for i, layer in enumerate(config["layers"]):
+            m, c, lw = layer["mixer"], self.layer_cfg[i], self.layer_w[i]
+            p, mp = f"l{i}.", f"l{i}.mix."
+            c.heads, c.dim, c.vdim, c.scale, c.kv_from = m["heads"], m["dim"], m["vdim"], m["scale"], -1
+            c.kv_heads = m.get("kv_heads", m["heads"])
+            c.rot_dims, c.rot_base = m["rot"]["dims"], m["rot"]["base"]
+            c.window = m["mask"]["size"] if m.get("mask") else 0
+            lw.norm1, lw.sinks = self._vector(weights[p + "norm1"]), self._vector(weights[mp + "sink"])
+            lw.out_proj = self._matrix([weights[mp + "o"]])
+            if layer["type"] == "attention":
+                c.mixer, c.tied_values = MIXERS["rotary"], 1
+                lw.in_proj = self._matrix([weights[mp + "q"], weights[mp + "k"]])
+            else:
+                c.mixer, c.head_gate = MIXERS["latent"], 1
+                c.q_rank, c.kv_rank, c.rot_part = m["q_rank"], m["kv_rank"], m["rot_dim"]
+                lw.in_proj = self._matrix([weights[mp + "dq"], weights[mp + "dkv"], weights[mp + "g"]])
+                lw.q_norm, lw.kv_norm = self._vector(weights[mp + "dq.norm"]), self._vector(weights[mp + "dkv.norm"])
+                lw.q_up = self._matrix([weights[mp + "uq"]])
+                rows = int(lib().w4a32_layered_head_rows(m["dim"], m["vdim"]))
+                lw.k_up = self._hold(pack_operand_blocks(weights[mp + "uk"].to(self.dtype), m["heads"], rows))
+                lw.v_up = self._hold(pack_operand_blocks(weights[mp + "uv"].to(self.dtype), m["heads"], rows))
+            if layer.get("mlp"):
+                r, e = layer["mlp"]["router"], layer["mlp"]["expert"]
+                c.experts, c.top, c.ff, c.expert_limit = r["experts"], r["top"], e["ff"], e["limit"]
+                lw.norm2, lw.router = self._vector(weights[p + "norm2"]), self._matrix([weights[p + "mlp.router"]])
+                of = lambda n: torch.stack([weights[f"{p}mlp.e{j}.{n}"].to(self.dtype) for j in range(c.experts)])
+                lw.gate_up = self._hold(pack_gate_up(of("gate"), of("up")))
+                down = torch.zeros((c.experts, _pad64(self.cfg.hidden), _pad64(c.ff)), dtype=self.dtype, device="cuda")
+                down[:, :self.cfg.hidden, :c.ff] = of("down")
+                lw.experts_down = self._hold(down)
+        W, Wp = self.cfg.hidden, _pad64(self.cfg.hidden)
+        loop_in = torch.zeros((Wp, 2, Wp), dtype=self.dtype, device="cuda")
+        loop_in[:W, :, :W] = weights["loop.in"].view(W, 2, W)
+        embed = self._matrix([weights["embed"]], False)
+        self.weights = LayeredWeights(embed, self._vector(weights["final.norm"]), embed, self.layer_w, self._hold(loop_in))
 
     def _hold(self, t):
         self._keep.append(t)

@@ -2,10 +2,15 @@
 // layered decoder. Host code only.
 //
 // A prefill layer:  [add + norm + input convolution] [in_proj] mixer [out_proj] [add + norm + input convolution] [up]
-//                   [PolyNorm] [down];  mixer = [convolution + cache append] [block means] [attention], or
-//                   [convolution] [chunks] [scan] [output] (retention: without the first)
+//                   [PolyNorm] [down];  mixer = [convolution or rotation + cache append] [block means] [attention], or
+//                   [convolution] [chunks] [scan] [output] (retention: without the first), or
+//                   [norms + cache append] [q_up] [expand] [attention];
+//                   a mixture of experts instead of the last three: [router] [choose] [plan] [gate, up] [down]
 // A decode layer:   [add + norm + input convolution + in_proj] [mixer step] [merge or head norm + gate + out_proj]
 //                   [add + norm + input convolution + up] [PolyNorm + down]
+//                   latent mixer: [norm + q_up] [cache append, query folded] [attention] [merge + values + gate] [out_proj]
+//                   mixture of experts: [add + norm + router] [norm + choice + gate, up] [down]
+// In front of a pass through looped layers: [add + loop_in].
 #include "w4a32_layered.h"
 
 #include <algorithm>
@@ -38,19 +43,39 @@ struct LayerGeom {
   int conv_rows;    // ... of which pass the short convolution
   int mix;          // heads * vdim
   int D, dv16;
-  int src, pool_owner;  // attention: whose keys and values, whose block means
-  int rot;              // retention: index of the rotation table, -1: none
+  int src, pool_owner;  // attention: whose keys and values, whose block means (runs)
+  int rot;              // index of the rotation table, -1: none
+  int q_rows;           // latent: heads * (dim + rot_part)
+  int Dc, Dr;           // latent: kv_rank and rot_part, padded
 };
+
+// One run of a layer; looped layers run several times, each time on caches of their own.
+struct LayerRun {
+  int layer;
+  bool pass_starts;  // the looped part's input product comes first
+};
+
+std::vector<LayerRun> layer_runs(const w4a32_layered_config* c) {
+  std::vector<LayerRun> r;
+  const bool loop = c->loop_times > 0;
+  for (int i = 0; i < (loop ? c->loop_start : c->n_layers); ++i) r.push_back({i, false});
+  if (!loop) return r;
+  for (int t = 0; t < c->loop_times; ++t)
+    for (int i = c->loop_start; i < c->loop_stop; ++i) r.push_back({i, i == c->loop_start});
+  for (int i = c->loop_stop; i < c->n_layers; ++i) r.push_back({i, false});
+  return r;
+}
 
 struct RotTable {
   int dims;
-  float base;
+  double base;
   size_t sin_off, cos_off;
 };
 
 struct Geom {
   int Hp, elem;
-  std::vector<LayerGeom> layers;
+  std::vector<LayerRun> runs;
+  std::vector<LayerGeom> layers;  // per run, as `st`
   std::vector<RotTable> rot;
   // state
   struct LayerState {
@@ -61,14 +86,27 @@ struct Geom {
   size_t state_bytes;
   // workspace
   size_t x[2], y, raw, cx, q, mix, parts, ff, z, o, ml, amax_v, amax_i, logits, last, rec, ws_bytes;
+  size_t cq, ke, ve, qa, head_out, router, moe, sel;  // latent attention, mixture of experts
+  std::vector<int> expand_blk;                        // per run: blocks of keys the expansion has room for
 };
+
+w4::MoeGeom moe_geom(const w4a32_layered_config* c, const w4a32_layer_config& l) {
+  return {c->hidden, pad64(c->hidden), l.ff, pad64(l.ff), l.experts, l.top, l.expert_limit};
+}
+constexpr int kRouterParts = 8;  // most parts a router product is dealt to
 
 int check_config(const w4a32_layered_config* c) {
   if (!c || !c->layers) return W4A32_EINVAL;
   if (c->hidden <= 0 || c->vocab <= 0 || c->n_layers <= 0 || c->max_seq <= 0 || c->max_batch_tokens <= 0)
     return W4A32_EINVAL;
   if (c->dtype != W4A32_LAYERED_BF16 && c->dtype != W4A32_LAYERED_F32) return W4A32_EINVAL;
-  if (c->canon_taps < 1 || !(c->norm_eps >= 0.0f)) return W4A32_EINVAL;
+  if (c->norm != W4A32_NORM_LAYER && c->norm != W4A32_NORM_RMS) return W4A32_EINVAL;
+  if (c->canon_taps < (c->norm == W4A32_NORM_RMS ? 0 : 1) || !(c->norm_eps >= 0.0f)) return W4A32_EINVAL;
+  if (c->loop_times < 0) return W4A32_EINVAL;
+  if (c->loop_times > 0) {
+    if (c->loop_start < 0 || c->loop_stop <= c->loop_start || c->loop_stop > c->n_layers) return W4A32_ESHAPE;
+    if (!w4::row_linear_fits(2 * pad64(c->hidden))) return W4A32_ENOTSUP;
+  }
   if (c->canon_taps > W4A32_LAYERED_MAX_TAPS) return W4A32_ENOTSUP;
   const int Hp = pad64(c->hidden);
   if (!w4::norm_conv_fits(Hp, c->canon_taps) || !w4::row_linear_fits(Hp)) return W4A32_ENOTSUP;
@@ -78,7 +116,11 @@ int check_config(const w4a32_layered_config* c) {
     if (l.heads % l.kv_heads != 0) return W4A32_ESHAPE;
     if (std::max(l.dim, l.vdim) > W4A32_LAYERED_MAX_DIM || l.conv_taps > W4A32_LAYERED_MAX_TAPS) return W4A32_ENOTSUP;
     if (!w4::row_linear_fits(pad64(l.heads * l.vdim))) return W4A32_ENOTSUP;
-    if (l.ff > 0 && (!w4::row_linear_fits(pad64(l.ff)) || !w4::polynorm_fits(pad64(l.ff)))) return W4A32_ENOTSUP;
+    if (l.ff > 0 && l.experts != 0) {
+      if (l.experts < 0 || l.top <= 0 || l.top > l.experts || !(l.expert_limit > 0.0f)) return W4A32_EINVAL;
+      if (l.experts > W4A32_LAYERED_MAX_EXPERTS || l.top > W4A32_LAYERED_MAX_TOP || !w4::moe_decode_fits(moe_geom(c, l)))
+        return W4A32_ENOTSUP;
+    } else if (l.ff > 0 && (!w4::row_linear_fits(pad64(l.ff)) || !w4::polynorm_fits(pad64(l.ff)))) return W4A32_ENOTSUP;
     switch (l.mixer) {
       case W4A32_MIX_ATTENTION: {
         if (l.window <= 0 || l.pool <= 0 || l.conv_taps < 0) return W4A32_EINVAL;
@@ -98,7 +140,23 @@ int check_config(const w4a32_layered_config* c) {
         break;
       case W4A32_MIX_RETENTION:
         if (l.kv_heads != l.heads || l.rot_dims < 0 || l.rot_dims % 2 != 0 || l.rot_dims > l.dim) return W4A32_ESHAPE;
-        if (l.rot_dims > 0 && !(l.rot_base > 0.0f)) return W4A32_EINVAL;
+        if (l.rot_dims > 0 && !(l.rot_base > 0.0)) return W4A32_EINVAL;
+        break;
+      case W4A32_MIX_ROTARY:
+        if (l.window < 0 || l.rot_dims < 0) return W4A32_EINVAL;
+        if (l.rot_dims % 2 != 0 || l.rot_dims > l.dim || (l.tied_values && l.vdim != l.dim)) return W4A32_ESHAPE;
+        if (l.rot_dims > 0 && !(l.rot_base > 0.0)) return W4A32_EINVAL;
+        if (l.conv_taps != 0 || l.heads / l.kv_heads * w4::head_bucket(std::max(l.dim, l.vdim)) > 4096 ||
+            l.heads / l.kv_heads > 32)
+          return W4A32_ENOTSUP;
+        break;
+      case W4A32_MIX_LATENT:
+        if (l.window < 0 || l.rot_dims < 0 || l.q_rank <= 0 || l.kv_rank <= 0 || l.rot_part < 0) return W4A32_EINVAL;
+        if (l.kv_heads != l.heads || l.rot_dims % 2 != 0 || l.rot_dims > l.rot_part) return W4A32_ESHAPE;
+        if (l.rot_dims > 0 && !(l.rot_base > 0.0)) return W4A32_EINVAL;
+        if (l.conv_taps != 0 || l.kv_rank > W4A32_LAYERED_MAX_LATENT || l.rot_part > W4A32_LAYERED_MAX_ROT_PART ||
+            !w4::row_linear_fits(pad64(l.q_rank)))
+          return W4A32_ENOTSUP;
         break;
       default: return W4A32_EINVAL;
     }
@@ -118,10 +176,18 @@ Geom geometry(const w4a32_layered_config* c) {
     o = align_up(o + bytes, 256);
     return at;
   };
-  int raw = 0, cx = 0, q = 0, mix = 0, ff = 0, ofl = 0, mlfl = 0;
-  size_t rec = 0;
-  for (int i = 0; i < c->n_layers; ++i) {
-    const w4a32_layer_config& l = c->layers[i];
+  int raw = 0, cx = 0, q = 0, mix = 0, ff = 0, z = 0, ofl = 0, mlfl = 0, cq = 0, qa = 0, head_out = 0, experts = 0;
+  size_t rec = 0, expand = 0, moe = 0, parts = g.Hp * Mb;
+  g.runs = layer_runs(c);
+  auto rot_table = [&](int dims, double base) {
+    if (dims == 0) return -1;
+    for (size_t r = 0; r < g.rot.size(); ++r)
+      if (g.rot[r].dims == dims && g.rot[r].base == base) return (int)r;
+    g.rot.push_back({dims, base, 0, 0});
+    return (int)g.rot.size() - 1;
+  };
+  for (int i = 0; i < (int)g.runs.size(); ++i) {
+    const w4a32_layer_config& l = c->layers[g.runs[i].layer];
     LayerGeom lg{};
     Geom::LayerState st{};
     lg.mix = l.heads * l.vdim;
@@ -129,13 +195,16 @@ Geom geometry(const w4a32_layered_config* c) {
     lg.dv16 = (l.vdim + 15) / 16 * 16;
     lg.src = lg.pool_owner = i;
     lg.rot = -1;
-    st.canon1 = take(sizeof(float) * c->canon_taps * g.Hp);
-    if (l.ff > 0) st.canon2 = take(sizeof(float) * c->canon_taps * g.Hp);
+    if (c->canon_taps > 0) st.canon1 = take(sizeof(float) * c->canon_taps * g.Hp);
+    if (l.ff > 0 && c->canon_taps > 0) st.canon2 = take(sizeof(float) * c->canon_taps * g.Hp);
     if (l.mixer == W4A32_MIX_ATTENTION) {
       lg.rows = lg.conv_rows = l.heads * l.dim + (l.kv_from < 0 ? l.kv_heads * (l.dim + l.vdim) : 0);
-      lg.src = l.kv_from >= 0 ? l.kv_from : i;
+      if (l.kv_from >= 0)  // the last run of that layer
+        for (int e = 0; e < i; ++e)
+          if (g.runs[e].layer == l.kv_from) lg.src = e;
       for (int e = 0; e < i; ++e) {
-        if (c->layers[e].mixer == W4A32_MIX_ATTENTION && g.layers[e].src == lg.src && c->layers[e].pool == l.pool) {
+        const w4a32_layer_config& le = c->layers[g.runs[e].layer];
+        if (le.mixer == W4A32_MIX_ATTENTION && g.layers[e].src == lg.src && le.pool == l.pool) {
           lg.pool_owner = g.layers[e].pool_owner;
           break;
         }
@@ -160,6 +229,35 @@ Geom geometry(const w4a32_layered_config* c) {
       q = std::max(q, l.heads * lg.D);
       ofl = std::max(ofl, w4::kPoolAttnSlices * l.heads * lg.D);
       mlfl = std::max(mlfl, w4::kPoolAttnSlices * l.heads * 2);
+    } else if (l.mixer == W4A32_MIX_ROTARY) {
+      lg.rows = l.heads * l.dim + l.kv_heads * (l.dim + (l.tied_values ? 0 : l.vdim));
+      st.cap = cap;
+      st.k = take((size_t)g.elem * l.kv_heads * cap * lg.D);
+      st.vt = take((size_t)g.elem * l.kv_heads * cap * lg.D);
+      lg.rot = rot_table(l.rot_dims, l.rot_base);
+      q = std::max(q, l.heads * lg.D);
+      ofl = std::max(ofl, w4::kPoolAttnSlices * l.heads * lg.D);
+      mlfl = std::max(mlfl, w4::kPoolAttnSlices * l.heads * 2);
+    } else if (l.mixer == W4A32_MIX_LATENT) {
+      lg.rows = l.q_rank + l.kv_rank + l.rot_part + (l.head_gate ? l.heads : 0);
+      lg.q_rows = l.heads * (l.dim + l.rot_part);
+      lg.Dc = pad64(l.kv_rank);
+      lg.Dr = w4::latent_rot_pad(l.rot_part);
+      st.cap = cap;
+      st.k = take((size_t)g.elem * cap * (lg.Dc + lg.Dr));
+      st.vt = take((size_t)g.elem * cap * lg.Dc);
+      lg.rot = rot_table(l.rot_dims, l.rot_base);
+      const int window = l.window > 0 ? l.window : w4::kNoWindow;
+      g.expand_blk.resize(g.runs.size(), 0);
+      g.expand_blk[i] = w4::latent_expand_blocks(window, c->max_seq, c->max_batch_tokens);
+      expand = std::max(expand, w4::latent_expand_elems(l.heads, lg.D, g.expand_blk[i]));
+      cq = std::max(cq, pad64(l.q_rank));
+      // (a decode step's query row is f32)
+      q = std::max(q, pad64(lg.q_rows) * (int)(sizeof(float) / g.elem));
+      qa = std::max(qa, l.heads * (lg.Dc + lg.Dr));
+      ofl = std::max(ofl, w4::kPoolAttnSlices * l.heads * lg.Dc);
+      mlfl = std::max(mlfl, w4::kPoolAttnSlices * l.heads * 2);
+      head_out = std::max(head_out, pad64(lg.mix));
     } else {
       const bool delta = l.mixer == W4A32_MIX_DELTA;
       const int nq = (delta ? l.kv_heads : l.heads) * l.dim;
@@ -168,13 +266,8 @@ Geom geometry(const w4a32_layered_config* c) {
       if (delta) {
         st.conv = take(sizeof(float) * l.conv_taps * pad64(lg.conv_rows));
         cx = std::max(cx, pad64(lg.conv_rows));
-      } else if (l.rot_dims > 0) {
-        for (size_t r = 0; r < g.rot.size(); ++r)
-          if (g.rot[r].dims == l.rot_dims && g.rot[r].base == l.rot_base) lg.rot = (int)r;
-        if (lg.rot < 0) {
-          lg.rot = (int)g.rot.size();
-          g.rot.push_back({l.rot_dims, l.rot_base, 0, 0});
-        }
+      } else {
+        lg.rot = rot_table(l.rot_dims, l.rot_base);
       }
       st.rec = take(sizeof(float) * (size_t)l.heads * lg.dv16 * lg.D);
       ofl = std::max(ofl, lg.mix);
@@ -182,7 +275,14 @@ Geom geometry(const w4a32_layered_config* c) {
     }
     raw = std::max(raw, pad64(lg.rows));
     mix = std::max(mix, pad64(lg.mix));
-    ff = std::max(ff, pad64(l.ff));
+    if (l.ff > 0 && l.experts > 0) {
+      experts = std::max(experts, l.experts);
+      z = std::max(z, l.top * pad64(l.ff));
+      moe = std::max(moe, w4::moe_scratch_bytes(c->dtype, c->max_batch_tokens, l.experts, l.top, pad64(l.ff)));
+      parts = std::max(parts, (size_t)l.top * Mb * g.Hp);
+    } else {
+      ff = std::max(ff, pad64(l.ff));
+    }
     g.layers.push_back(lg);
     g.st.push_back(st);
   }
@@ -195,14 +295,14 @@ Geom geometry(const w4a32_layered_config* c) {
   }
   g.x[0] = take(sizeof(float) * Mb * g.Hp);
   g.x[1] = take(sizeof(float) * Mb * g.Hp);
-  g.y = take((size_t)g.elem * Mb * g.Hp);
+  g.y = take((size_t)g.elem * Mb * g.Hp * (c->loop_times > 0 ? 2 : 1));
   g.raw = take(sizeof(float) * Mb * raw);
   g.cx = take(sizeof(float) * Mb * cx);
   g.q = take((size_t)g.elem * Mb * q);
   g.mix = take((size_t)g.elem * Mb * mix);
-  g.parts = take(sizeof(float) * std::max(Mb * g.Hp, kSplitFloats));
+  g.parts = take(sizeof(float) * std::max(parts, kSplitFloats));
   g.ff = take((size_t)g.elem * Mb * ff);
-  g.z = take(sizeof(float) * ff);
+  g.z = take(sizeof(float) * std::max(ff, z));
   g.o = take(sizeof(float) * ofl);
   g.ml = take(sizeof(float) * mlfl);
   g.amax_v = take(sizeof(float) * kArgmaxParts);
@@ -210,6 +310,14 @@ Geom geometry(const w4a32_layered_config* c) {
   g.logits = take(sizeof(float) * c->vocab);
   g.last = take(sizeof(int));
   g.rec = take(sizeof(float) * rec);
+  g.cq = take((size_t)g.elem * Mb * cq);
+  g.ke = take(g.elem * expand);
+  g.ve = take(g.elem * expand);
+  g.qa = take(sizeof(float) * qa);
+  g.head_out = take(sizeof(float) * head_out);
+  g.router = take(sizeof(float) * kRouterParts * Mb * pad64(experts));
+  g.moe = take(moe);
+  g.sel = take(sizeof(int) * W4A32_LAYERED_MAX_TOP);
   g.ws_bytes = o;
   return g;
 }
@@ -226,10 +334,30 @@ struct Run {
   float* stf(size_t off) const { return reinterpret_cast<float*>(st + off); }
   int* pos() const { return reinterpret_cast<int*>(st); }
   bool bf16() const { return c->dtype == W4A32_LAYERED_BF16; }
+  // of run i
+  const w4a32_layer_config& layer(int i) const { return c->layers[g.runs[i].layer]; }
+  const w4a32_layered_layer& weights(int i) const { return w->layers[g.runs[i].layer]; }
+  w4::NormSpec norm_spec() const {
+    return {c->norm_eps, c->residual_mult != 0.0f ? c->residual_mult : 1.0f, c->norm == W4A32_NORM_RMS};
+  }
+  const float *sin_t(int i) const { return g.layers[i].rot >= 0 ? f32(g.rot[g.layers[i].rot].sin_off) : nullptr; }
+  const float *cos_t(int i) const { return g.layers[i].rot >= 0 ? f32(g.rot[g.layers[i].rot].cos_off) : nullptr; }
 
   w4::AttnGeom attn_geom(int i) const {
-    const w4a32_layer_config& l = c->layers[i];
+    const w4a32_layer_config& l = layer(i);
     w4::AttnGeom a{};
+    if (l.mixer == W4A32_MIX_ROTARY) {
+      a.heads = l.heads; a.kv_heads = l.kv_heads; a.dim = l.dim; a.vdim = l.vdim; a.D = g.layers[i].D;
+      a.cap = g.st[i].cap; a.capp = 32;
+      a.window = l.window > 0 ? l.window : w4::kNoWindow;
+      a.scale = l.scale;
+      a.own_kv = true;
+      a.tied = l.tied_values != 0;
+      a.rot_dims = l.rot_dims; a.rot_rows = c->max_seq;
+      a.sin_t = sin_t(i); a.cos_t = cos_t(i);
+      a.sinks = weights(i).sinks;
+      return a;
+    }
     a.heads = l.heads; a.kv_heads = l.kv_heads; a.dim = l.dim; a.vdim = l.vdim; a.D = g.layers[i].D;
     a.cap = g.st[i].cap; a.capp = g.st[i].capp;
     a.window = l.window; a.pool = l.pool; a.scale = l.scale;
@@ -240,11 +368,32 @@ struct Run {
   }
   w4::AttnMem attn_mem(int i) const {
     const auto& t = g.st[i];
-    return {st + t.k, st + t.vt, st + t.kp, st + t.vpt, c->layers[i].conv_taps > 0 ? stf(t.conv) : nullptr};
+    return {st + t.k, st + t.vt, st + t.kp, st + t.vpt, layer(i).conv_taps > 0 ? stf(t.conv) : nullptr};
+  }
+  w4::LatentGeom latent_geom(int i) const {
+    const w4a32_layer_config& l = layer(i);
+    const w4a32_layered_layer& lw = weights(i);
+    const LayerGeom& lg = g.layers[i];
+    w4::LatentGeom a{};
+    a.heads = l.heads; a.dim = l.dim; a.vdim = l.vdim; a.D = lg.D;
+    a.q_rank = l.q_rank; a.kv_rank = l.kv_rank; a.rot_part = l.rot_part;
+    a.Dc = lg.Dc; a.Dr = lg.Dr;
+    a.cap = g.st[i].cap;
+    a.window = l.window > 0 ? l.window : w4::kNoWindow;
+    a.ldr = pad64(lg.rows);
+    a.kv_off = l.q_rank; a.rot_off = l.q_rank + l.kv_rank;
+    a.gate_off = l.head_gate ? a.rot_off + l.rot_part : -1;
+    a.scale = l.scale;
+    a.eps = c->norm_eps;
+    a.rot_dims = l.rot_dims; a.rot_rows = c->max_seq;
+    a.sin_t = sin_t(i); a.cos_t = cos_t(i);
+    a.sinks = lw.sinks; a.q_norm = lw.q_norm; a.kv_norm = lw.kv_norm;
+    a.k_up = lw.k_up; a.v_up = lw.v_up;
+    return a;
   }
   w4::RecGeom rec_geom(int i) const {
-    const w4a32_layer_config& l = c->layers[i];
-    const w4a32_layered_layer& lw = w->layers[i];
+    const w4a32_layer_config& l = layer(i);
+    const w4a32_layered_layer& lw = weights(i);
     w4::RecGeom r{};
     r.delta = l.mixer == W4A32_MIX_DELTA;
     r.heads = l.heads; r.kv_heads = l.kv_heads; r.dim = l.dim; r.vdim = l.vdim; r.D = g.layers[i].D;
@@ -257,8 +406,8 @@ struct Run {
     r.a_log = lw.a_log; r.dt_bias = lw.dt_bias; r.head_norm = r.delta ? lw.head_norm : nullptr;
     r.decay = lw.decay; r.log_decay = lw.log_decay;
     if (g.layers[i].rot >= 0) {
-      r.sin_t = f32(g.rot[g.layers[i].rot].sin_off);
-      r.cos_t = f32(g.rot[g.layers[i].rot].cos_off);
+      r.sin_t = sin_t(i);
+      r.cos_t = cos_t(i);
       r.rot_dims = l.rot_dims;
     }
     r.rot_rows = c->max_seq;
@@ -285,22 +434,38 @@ int prefill_layers(const Run& r, const int64_t* tokens, int M, int pos0, int n_l
   const int H = c->hidden, Hp = g.Hp, dt = c->dtype;
   int cur = 0, pending = 0;
   W4_LAUNCH(w4::launch_embed_rows(dt, tokens, r.w->embedding, M, H, Hp, c->vocab, r.f32(g.x[0]), r.s));
+  const w4::NormSpec spec = r.norm_spec();
   auto norm = [&](const float* w, const float* conv, size_t ring) {
     const int rc = from_hip(w4::launch_norm_conv(r.f32(g.x[cur]), r.f32(g.parts), pending, r.f32(g.x[cur ^ 1]), w,
-                                                 c->norm_eps, conv, r.stf(ring), c->canon_taps, M, H, Hp, pos0,
+                                                 spec, conv, r.stf(ring), c->canon_taps, M, H, Hp, pos0,
                                                  r.ws + g.y, r.bf16(), r.s));
     if (pending) cur ^= 1;
     pending = 0;
     return rc;
   };
   for (int i = 0; i < n_layers; ++i) {
-    const w4a32_layer_config& l = c->layers[i];
-    const w4a32_layered_layer& lw = r.w->layers[i];
+    const w4a32_layer_config& l = r.layer(i);
+    const w4a32_layered_layer& lw = r.weights(i);
     const LayerGeom& lg = g.layers[i];
     const int ldr = pad64(lg.rows), ldm = pad64(lg.mix);
+    if (g.runs[i].pass_starts) {
+      W4_LAUNCH(w4::launch_loop_rows(dt, r.f32(g.x[cur]), r.f32(g.parts), pending, spec.part_scale, tokens, r.w->embedding,
+                                     c->vocab, M, Hp, r.ws + g.y, r.s));
+      W4_TRY(product(r, r.ws + g.y, r.w->loop_in, r.f32(g.x[cur]), M, Hp, 2 * Hp, false, nullptr));
+      pending = 0;
+    }
     W4_TRY(norm(lw.norm1, lw.canon1, g.st[i].canon1));
     W4_TRY(product(r, r.ws + g.y, lw.in_proj, r.f32(g.raw), M, ldr, Hp, false, nullptr));
-    if (l.mixer == W4A32_MIX_ATTENTION) {
+    if (l.mixer == W4A32_MIX_LATENT) {
+      const w4::LatentGeom a = r.latent_geom(i);
+      uint8_t *k = r.st + g.st[i].k, *vt = r.st + g.st[i].vt;
+      const int ldc = pad64(l.q_rank), ldq = pad64(lg.q_rows), nblk = g.expand_blk[i];
+      W4_LAUNCH(w4::launch_latent_rows(dt, a, k, vt, r.f32(g.raw), r.ws + g.cq, ldc, M, pos0, r.s));
+      W4_TRY(product(r, r.ws + g.cq, lw.q_up, r.ws + g.q, M, ldq, ldc, true, nullptr));
+      W4_LAUNCH(w4::launch_latent_expand(dt, a, k, r.ws + g.ke, r.ws + g.ve, nblk, M, pos0, r.s));
+      W4_LAUNCH(w4::launch_latent_prefill(dt, a, k, r.ws + g.ke, r.ws + g.ve, nblk, r.ws + g.q, ldq, r.f32(g.raw),
+                                          r.ws + g.mix, ldm, M, pos0, r.s));
+    } else if (l.mixer == W4A32_MIX_ATTENTION || l.mixer == W4A32_MIX_ROTARY) {
       const w4::AttnGeom a = r.attn_geom(i);
       const w4::AttnMem m = r.attn_mem(i);
       W4_LAUNCH(w4::launch_attn_qkv(dt, a, m, r.f32(g.raw), ldr, l.conv_taps > 0 ? lw.conv : nullptr, r.ws + g.q, M,
@@ -318,7 +483,20 @@ int prefill_layers(const Run& r, const int64_t* tokens, int M, int pos0, int n_l
                                        r.ws + g.mix, ldm, M, pos0, r.s));
     }
     W4_TRY(product(r, r.ws + g.mix, lw.out_proj, r.f32(g.parts), M, Hp, ldm, false, &pending));
-    if (l.ff > 0) {
+    if (l.ff > 0 && l.experts > 0) {
+      const int Ep = pad64(l.experts);
+      W4_TRY(norm(lw.norm2, lw.canon2, g.st[i].canon2));
+      int rp = 1;  // few tiles: dealt over k as far as that goes
+      if (r.bf16()) {
+        rp = std::max(1, std::min(kRouterParts, Hp / 128));
+        W4_LAUNCH(w4::launch_matmul_bf16(r.ws + g.y, lw.router, r.f32(g.router), M, Ep, Hp, Ep, false, rp, r.s));
+      } else {
+        W4_TRY(product(r, r.ws + g.y, lw.router, r.f32(g.router), M, Ep, Hp, false, nullptr));
+      }
+      W4_LAUNCH(w4::launch_moe_prefill(dt, moe_geom(c, l), r.ws + g.y, r.f32(g.router), rp, Ep, lw.gate_up, lw.experts_down, M,
+                                       r.f32(g.parts), r.ws + g.moe, r.s));
+      pending = l.top;
+    } else if (l.ff > 0) {
       const int Fp = pad64(l.ff);
       W4_TRY(norm(lw.norm2, lw.canon2, g.st[i].canon2));
       W4_TRY(product(r, r.ws + g.y, lw.up, r.ws + g.ff, M, Fp, Hp, true, nullptr));
@@ -339,21 +517,33 @@ int decode_layers(const Run& r, const int64_t* token, int n_layers, int* cur_out
   int cur = 0, pending = 0;
   float* raw = r.f32(g.raw);
   float* part = r.f32(g.parts);
+  const w4::NormSpec spec = r.norm_spec();
   for (int i = 0; i < n_layers; ++i) {
-    const w4a32_layer_config& l = c->layers[i];
-    const w4a32_layered_layer& lw = r.w->layers[i];
+    const w4a32_layer_config& l = r.layer(i);
+    const w4a32_layered_layer& lw = r.weights(i);
     const LayerGeom& lg = g.layers[i];
     w4::RowPrologue p{};
     p.K = c->hidden;
     p.x = r.f32(g.x[cur]);
-    if (i == 0) {
-      p.token = token;
-      p.table = r.w->embedding;
-      p.vocab = c->vocab;
-    }
+    p.table = r.w->embedding;
+    p.vocab = c->vocab;
     p.parts = part;
     p.n_parts = pending;
     p.part_stride = Hp;
+    p.part_scale = spec.part_scale;
+    p.rms = spec.rms;
+    if (g.runs[i].pass_starts) {
+      w4::RowPrologue q = p;
+      q.token = token;
+      if (i == 0) q.x = nullptr;
+      W4_LAUNCH(w4::launch_row_linear(w4::kRowLoop, dt, q, r.w->loop_in, Hp, 2 * Hp, r.f32(g.x[cur ^ 1]), nullptr, nullptr,
+                                      r.s));
+      cur ^= 1;
+      p.x = r.f32(g.x[cur]);
+      p.n_parts = 0;
+    } else if (i == 0) {
+      p.token = token;
+    }
     p.x_out = r.f32(g.x[cur ^ 1]);
     p.norm_w = lw.norm1;
     p.eps = c->norm_eps;
@@ -371,7 +561,23 @@ int decode_layers(const Run& r, const int64_t* token, int n_layers, int* cur_out
     m.vdim = l.vdim;
     m.eps = c->norm_eps;
     int kind;
-    if (l.mixer == W4A32_MIX_ATTENTION) {
+    if (l.mixer == W4A32_MIX_LATENT) {
+      const w4::LatentGeom a = r.latent_geom(i);
+      void *k = r.st + g.st[i].k, *vt = r.st + g.st[i].vt;
+      float *q = r.f32(g.q), *qa = r.f32(g.qa), *o = r.f32(g.o), *ml = r.f32(g.ml);
+      w4::RowPrologue n{};
+      n.K = l.q_rank;
+      n.x = raw;
+      n.norm_w = lw.q_norm;
+      n.eps = c->norm_eps;
+      n.rms = true;
+      W4_LAUNCH(w4::launch_row_linear(w4::kRowNorm, dt, n, lw.q_up, lg.q_rows, pad64(l.q_rank), q, nullptr, nullptr, r.s));
+      W4_LAUNCH(w4::launch_latent_absorb(dt, a, k, vt, raw, q, r.pos(), qa, r.s));
+      W4_LAUNCH(w4::launch_latent_decode(dt, a, k, vt, qa, r.pos(), c->max_seq, o, ml, r.s));
+      W4_LAUNCH(w4::launch_latent_out(dt, a, o, ml, w4::latent_slices(a.window, c->max_seq), raw, r.f32(g.head_out), r.s));
+      m.x = r.f32(g.head_out);
+      kind = w4::kRowPlain;
+    } else if (l.mixer == W4A32_MIX_ATTENTION || l.mixer == W4A32_MIX_ROTARY) {
       W4_LAUNCH(w4::launch_attn_decode(dt, r.attn_geom(i), r.attn_mem(i), raw, lw.conv, r.pos(), c->max_seq,
                                        r.f32(g.o), r.f32(g.ml), r.s));
       m.ml = r.f32(g.ml);
@@ -397,6 +603,17 @@ int decode_layers(const Run& r, const int64_t* token, int n_layers, int* cur_out
       p.norm_w = lw.norm2;
       p.conv = lw.canon2;
       p.ring = r.stf(g.st[i].canon2);
+    }
+    if (l.ff > 0 && l.experts > 0) {
+      W4_LAUNCH(w4::launch_row_linear(w4::kRowNorm, dt, p, lw.router, l.experts, Hp, r.f32(g.router), nullptr, nullptr, r.s));
+      cur ^= 1;
+      // the completed residual row is there now (an input convolution's ring is written with the same row again)
+      p.x = r.f32(g.x[cur]);
+      p.n_parts = 0;
+      p.x_out = nullptr;
+      W4_LAUNCH(w4::launch_moe_decode(dt, moe_geom(c, l), p, r.f32(g.router), lw.gate_up, lw.experts_down, r.f32(g.z),
+                                      reinterpret_cast<int*>(r.ws + g.sel), part, r.s));
+    } else if (l.ff > 0) {
       W4_LAUNCH(w4::launch_row_linear(w4::kRowNorm, dt, p, lw.up, pad64(l.ff), Hp, r.f32(g.z), nullptr, nullptr, r.s));
       cur ^= 1;
       w4::RowPrologue f{};
@@ -421,6 +638,8 @@ int head_row(const Run& r, int cur, int pending, int row, int M, float* logits) 
   p.parts = r.f32(g.parts) + (size_t)row * g.Hp;
   p.n_parts = pending;
   p.part_stride = (size_t)M * g.Hp;
+  p.part_scale = r.norm_spec().part_scale;
+  p.rms = r.norm_spec().rms;
   p.norm_w = r.w->final_norm;
   p.eps = r.c->norm_eps;
   return from_hip(w4::launch_row_linear(w4::kRowNorm, r.c->dtype, p, r.w->head, r.c->vocab, g.Hp, logits,
@@ -436,14 +655,19 @@ int check_call(const w4a32_layered_config* c, const w4a32_layered_weights* w, co
   W4_TRY(check_config(c));
   if (!w || !w->embedding || !w->final_norm || !w->head || !w->layers || !st || !ws) return W4A32_EINVAL;
   if ((reinterpret_cast<uintptr_t>(st) & 255) != 0 || (reinterpret_cast<uintptr_t>(ws) & 255) != 0) return W4A32_EINVAL;
+  if (c->loop_times > 0 && !w->loop_in) return W4A32_EINVAL;
   for (int i = 0; i < c->n_layers; ++i) {
     const w4a32_layer_config& l = c->layers[i];
     const w4a32_layered_layer& lw = w->layers[i];
-    if (!lw.norm1 || !lw.canon1 || !lw.in_proj || !lw.out_proj) return W4A32_EINVAL;
+    if (!lw.norm1 || !lw.in_proj || !lw.out_proj) return W4A32_EINVAL;
+    if (c->canon_taps > 0 && (!lw.canon1 || (l.ff > 0 && !lw.canon2))) return W4A32_EINVAL;
+    if (l.mixer == W4A32_MIX_LATENT && (!lw.q_norm || !lw.kv_norm || !lw.q_up || !lw.k_up || !lw.v_up)) return W4A32_EINVAL;
     if (l.mixer != W4A32_MIX_RETENTION && l.conv_taps > 0 && !lw.conv) return W4A32_EINVAL;
     if (l.mixer == W4A32_MIX_DELTA && (!lw.a_log || !lw.dt_bias || !lw.head_norm)) return W4A32_EINVAL;
     if (l.mixer == W4A32_MIX_RETENTION && (!lw.decay || !lw.log_decay)) return W4A32_EINVAL;
-    if (l.ff > 0 && (!lw.norm2 || !lw.canon2 || !lw.up || !lw.down || !lw.act)) return W4A32_EINVAL;
+    if (l.ff > 0 && !lw.norm2) return W4A32_EINVAL;
+    if (l.ff > 0 && l.experts == 0 && (!lw.up || !lw.down || !lw.act)) return W4A32_EINVAL;
+    if (l.ff > 0 && l.experts > 0 && (!lw.router || !lw.gate_up || !lw.experts_down)) return W4A32_EINVAL;
   }
   return W4A32_OK;
 }
@@ -453,6 +677,12 @@ int check_call(const w4a32_layered_config* c, const w4a32_layered_weights* w, co
 extern "C" {
 
 int w4a32_layered_check(const w4a32_layered_config* cfg) { return check_config(cfg); }
+
+int w4a32_layered_head_rows(int dim, int vdim) { return w4::head_bucket(std::max(dim, vdim)); }
+
+int w4a32_layered_runs(const w4a32_layered_config* cfg) {
+  return check_config(cfg) == W4A32_OK ? (int)layer_runs(cfg).size() : 0;
+}
 
 size_t w4a32_layered_state_bytes(const w4a32_layered_config* cfg) {
   return check_config(cfg) == W4A32_OK ? geometry(cfg).state_bytes : 0;
@@ -497,11 +727,11 @@ int w4a32_layered_forward(const w4a32_layered_config* cfg, const w4a32_layered_w
   if (!d_tokens || n_tokens <= 0 || pos0 < 0 || n_want < 0 || stop_after < 0) return W4A32_EINVAL;
   if (n_want > 0 && (!d_want || !d_logits)) return W4A32_EINVAL;
   if (n_tokens > cfg->max_batch_tokens || n_want > n_tokens || pos0 > cfg->max_seq - n_tokens ||
-      stop_after > cfg->n_layers)
+      stop_after > (int)layer_runs(cfg).size())
     return W4A32_ESHAPE;
   const Geom g = geometry(cfg);
   const Run r{cfg, w, g, static_cast<uint8_t*>(d_state), static_cast<uint8_t*>(d_ws), S(stream)};
-  const int n_layers = stop_after > 0 ? stop_after : cfg->n_layers;
+  const int n_layers = stop_after > 0 ? stop_after : (int)g.runs.size();
   int cur = 0, pending = 0;
   if (n_tokens == 1) {
     W4_LAUNCH(w4::launch_set_int(r.pos(), pos0, r.s));
@@ -511,11 +741,11 @@ int w4a32_layered_forward(const w4a32_layered_config* cfg, const w4a32_layered_w
   }
   W4_LAUNCH(w4::launch_set_int(r.pos(), pos0 + n_tokens, r.s));
   if (stop_after > 0) {
-    return from_hip(w4::launch_add_parts(r.f32(g.x[cur]), r.f32(g.parts), pending, r.f32(g.x[0]), n_tokens, g.Hp, r.s));
+    return from_hip(w4::launch_add_parts(r.f32(g.x[cur]), r.f32(g.parts), pending, r.norm_spec().part_scale, r.f32(g.x[0]), n_tokens, g.Hp, r.s));
   }
   if (n_want == 0) return W4A32_OK;
   if (n_tokens == 1) return head_row(r, cur, pending, 0, 1, d_logits);
-  W4_LAUNCH(w4::launch_norm_want(r.f32(g.x[cur]), r.f32(g.parts), pending, w->final_norm, cfg->norm_eps, d_want, n_want,
+  W4_LAUNCH(w4::launch_norm_want(r.f32(g.x[cur]), r.f32(g.parts), pending, w->final_norm, r.norm_spec(), d_want, n_want,
                                  n_tokens, cfg->hidden, g.Hp, r.ws + g.y, r.bf16(), r.s));
   return product(r, r.ws + g.y, w->head, d_logits, n_want, cfg->vocab, g.Hp, false, nullptr);
 }
@@ -531,9 +761,9 @@ int w4a32_layered_prefill(const w4a32_layered_config* cfg, const w4a32_layered_w
   int cur = 0, pending = 0;
   if (n_tokens == 1) {
     W4_LAUNCH(w4::launch_set_int(r.pos(), pos0, r.s));
-    W4_TRY(decode_layers(r, d_tokens, cfg->n_layers, &cur, &pending));
+    W4_TRY(decode_layers(r, d_tokens, (int)g.runs.size(), &cur, &pending));
   } else {
-    W4_TRY(prefill_layers(r, d_tokens, n_tokens, pos0, cfg->n_layers, &cur, &pending));
+    W4_TRY(prefill_layers(r, d_tokens, n_tokens, pos0, (int)g.runs.size(), &cur, &pending));
   }
   W4_LAUNCH(w4::launch_set_int(r.pos(), pos0 + n_tokens, r.s));
   W4_TRY(head_row(r, cur, pending, n_tokens - 1, n_tokens, r.f32(g.logits)));
@@ -547,7 +777,7 @@ int w4a32_layered_step(const w4a32_layered_config* cfg, const w4a32_layered_weig
   const Geom g = geometry(cfg);
   const Run r{cfg, w, g, static_cast<uint8_t*>(d_state), static_cast<uint8_t*>(d_ws), S(stream)};
   int cur = 0, pending = 0;
-  W4_TRY(decode_layers(r, d_token_in, cfg->n_layers, &cur, &pending));
+  W4_TRY(decode_layers(r, d_token_in, (int)g.runs.size(), &cur, &pending));
   W4_TRY(head_row(r, cur, pending, 0, 1, r.f32(g.logits)));
   return pick_token(r, d_token_out, r.pos());
 }
@@ -567,7 +797,8 @@ int w4a32_op_layernorm_conv(const float* d_x, const float* d_parts, int n_parts,
   if (n_parts > 0 && (!d_parts || !d_x_out || d_x_out == d_x)) return W4A32_EINVAL;
   if (taps > 0 && (!d_conv || !d_ring)) return W4A32_EINVAL;
   if (taps > W4A32_LAYERED_MAX_TAPS || !w4::norm_conv_fits(pad64(H), taps)) return W4A32_ENOTSUP;
-  return from_hip(w4::launch_norm_conv(d_x, d_parts, n_parts, d_x_out, d_norm, eps, d_conv, d_ring, taps, M, H, pad64(H),
+  w4::NormSpec spec{eps};
+  return from_hip(w4::launch_norm_conv(d_x, d_parts, n_parts, d_x_out, d_norm, spec, d_conv, d_ring, taps, M, H, pad64(H),
                                        pos0, d_y, y_bf16 != 0, S(stream)));
 }
 
@@ -578,6 +809,23 @@ int w4a32_op_short_conv(const float* d_x, int ldx, float* d_y, int ldy, const fl
   if (ldx < channels || ldy < channels || ldw < channels) return W4A32_ESHAPE;
   return from_hip(w4::launch_short_conv(d_x, ldx, d_y, ldy, d_w, d_ring, ldw, taps, channels, apply_silu != 0, M, pos0,
                                         S(stream)));
+}
+
+size_t w4a32_op_experts_scratch_bytes(int dtype, int M, int experts, int top, int ff) {
+  if (M <= 0 || experts <= 0 || top <= 0 || ff <= 0) return 0;
+  return w4::moe_scratch_bytes(dtype, M, experts, top, pad64(ff));
+}
+
+int w4a32_op_experts(int dtype, const void* d_h, const float* d_logits, int ld, const void* d_gate_up, const void* d_down,
+                     int M, int hidden, int experts, int top, int ff, float limit, float* d_parts, void* d_scratch,
+                     void* stream) {
+  if (!d_h || !d_logits || !d_gate_up || !d_down || !d_parts || !d_scratch || M <= 0 || hidden <= 0 || experts <= 0 ||
+      top <= 0 || ff <= 0 || !(limit > 0.0f) || (dtype != W4A32_LAYERED_BF16 && dtype != W4A32_LAYERED_F32))
+    return W4A32_EINVAL;
+  if (top > experts || ld < experts) return W4A32_ESHAPE;
+  if (experts > W4A32_LAYERED_MAX_EXPERTS || top > W4A32_LAYERED_MAX_TOP) return W4A32_ENOTSUP;
+  const w4::MoeGeom g{hidden, pad64(hidden), ff, pad64(ff), experts, top, limit};
+  return from_hip(w4::launch_moe_prefill(dtype, g, d_h, d_logits, 1, ld, d_gate_up, d_down, M, d_parts, d_scratch, S(stream)));
 }
 
 int w4a32_op_polynorm(void* d_z, int z_bf16, int M, int F, int ld, const float* d_act, float eps, void* stream) {

@@ -69,6 +69,8 @@ enum RowKind {
   kRowMerge = 1,  // attention output from its key slices
   kRowGated = 2,  // per head: over its root mean square, times a weight, times silu(gate)
   kRowPoly = 3,   // PolyNorm
+  kRowPlain = 4,  // the row as it is
+  kRowLoop = 5,   // residual add of partial rows, the token's embedding row behind it (K: twice the padded width)
 };
 struct RowPrologue {
   int K;                // true length of the row
@@ -80,6 +82,8 @@ struct RowPrologue {
   const float* parts;   // n_parts partial rows, part_stride floats apart
   int n_parts;
   size_t part_stride;
+  float part_scale;     // factor of the partial rows
+  bool rms;             // divided by the root mean square, no mean taken off
   float* x_out;         // [ld], stored by the first workgroup
   const float* norm_w;
   float eps;
@@ -96,6 +100,7 @@ struct RowPrologue {
   const float* head_w;
   // kRowPoly: x is the row
   const float* act;
+  // kRowLoop: the residual row is x, or, without it, the embedding row as well
 };
 
 // y[n] = sum_k row[k] W[n][k], f32 output; W T [N][Kp]; optionally one (max, first column) pair per wavefront
@@ -113,14 +118,23 @@ int matmul_bf16_parts(int M, int N, int K);  // parts worth using for few tiles
 hipError_t launch_embed_rows(int dtype, const int64_t* ids, const void* table, int M, int H, int ld, int vocab,
                              float* x, hipStream_t s);
 bool norm_conv_fits(int ld, int taps);
+// how a residual row takes in the partial rows behind it, and how it is normed
+struct NormSpec {
+  float eps, part_scale = 1.0f;
+  bool rms = false;
+};
 hipError_t launch_norm_conv(const float* x, const float* parts, int n_parts, float* x_out, const float* norm_w,
-                            float eps, const float* conv, float* ring, int taps, int M, int H, int ld, int pos0,
+                            const NormSpec& spec, const float* conv, float* ring, int taps, int M, int H, int ld, int pos0,
                             void* y, bool y_bf16, hipStream_t s);
 // layer norm of the wanted rows (x + parts), no convolution: y [n_want][ld]
-hipError_t launch_norm_want(const float* x, const float* parts, int n_parts, const float* norm_w, float eps,
-                            const int* want, int n_want, int M, int H, int ld, void* y, bool y_bf16, hipStream_t s);
-// out = x + parts; out may be x
-hipError_t launch_add_parts(const float* x, const float* parts, int n_parts, float* out, int M, int ld, hipStream_t s);
+hipError_t launch_norm_want(const float* x, const float* parts, int n_parts, const float* norm_w,
+                            const NormSpec& spec, const int* want, int n_want, int M, int H, int ld, void* y, bool y_bf16, hipStream_t s);
+// out = x + scale * parts; out may be x
+hipError_t launch_add_parts(const float* x, const float* parts, int n_parts, float scale, float* out, int M, int ld,
+                            hipStream_t s);
+// y [M][2 ld] = [x + scale * parts, embedding row], element type T
+hipError_t launch_loop_rows(int dtype, const float* x, const float* parts, int n_parts, float scale, const int64_t* ids,
+                            const void* table, int vocab, int M, int ld, void* y, hipStream_t s);
 bool polynorm_fits(int ld);
 hipError_t launch_polynorm(void* z, bool z_bf16, int M, int F, int ld, const float* act, float eps, hipStream_t s);
 
@@ -141,7 +155,13 @@ struct AttnGeom {
   int ldc;              // leading dimension of the convolution's weights and ring
   bool own_kv;          // this layer projects keys and values itself
   bool make_pool;       // ... and / or is the one that keeps the block means it reads
+  bool tied;            // the values are the keys before rotation
+  int rot_dims, rot_rows;      // rotation of q and k (no convolution with it); rows of the tables
+  const float *sin_t, *cos_t;  // [rot_rows][rot_dims / 2]
+  const float* sinks;          // [heads], or null
 };
+constexpr int kNoWindow = 1 << 30;  // window of a layer that sees every token
+// pool 0: no block means
 struct AttnMem {
   void *k, *vt, *kp, *vpt;
   float* ring;
@@ -158,6 +178,58 @@ constexpr int kPoolAttnSlices = 16;  // most of them
 int attn_slices(const AttnGeom& g, int max_seq);
 hipError_t launch_attn_decode(int dtype, const AttnGeom& g, const AttnMem& m, const float* raw, const float* conv,
                               const int* pos, int max_seq, float* o, float* ml, hipStream_t s);
+
+// ---- latent attention ----
+// Cache of one layer: k [blocks][(Dc + Dr) / 8][32][8] holds a token's latent and rotated key part, vt [blocks][Dc][32] the
+// latent once more in the values' order (both as in w4a32_pooled_attention.hip, one kv head).
+struct LatentGeom {
+  int heads, dim, vdim, D;      // D = head_bucket(max(dim, vdim)): rows per head of the operand blocks
+  int q_rank, kv_rank, rot_part;
+  int Dc, Dr;                   // kv_rank padded to 64, rot_part to 16
+  int cap, window;
+  int ldr, kv_off, rot_off, gate_off;  // in_proj row: where the kv latent, the key part and the gates are (gate_off -1: none)
+  float scale, eps;
+  int rot_dims, rot_rows;
+  const float *sin_t, *cos_t, *sinks, *q_norm, *kv_norm;
+  const void *k_up, *v_up;
+};
+int latent_rot_pad(int rot_part);
+size_t latent_expand_elems(int heads, int D, int blocks);  // of each, keys and values
+int latent_expand_blocks(int window, int max_seq, int max_batch_tokens);
+// rows of a portion: the query's latent, normed, -> T cq [M][ldq]; latent and key part -> cache
+hipError_t launch_latent_rows(int dtype, const LatentGeom& g, void* k, void* vt, const float* raw, void* cq, int ldq, int M,
+                              int pos0, hipStream_t s);
+// keys and values of the tokens the portion sees -> ke, ve (nblk blocks allotted per head)
+hipError_t launch_latent_expand(int dtype, const LatentGeom& g, const void* k, void* ke, void* ve, int nblk, int M, int pos0,
+                                hipStream_t s);
+// q T [M][ldq], not yet rotated; out T [M][ldo]
+hipError_t launch_latent_prefill(int dtype, const LatentGeom& g, const void* k, const void* ke, const void* ve, int nblk,
+                                 const void* q, int ldq, const float* raw, void* out, int ldo, int M, int pos0,
+                                 hipStream_t s);
+// one token: cache append, q [heads * (dim + rot_part)] folded into the latent space -> qa f32 [heads][Dc + Dr]
+hipError_t launch_latent_absorb(int dtype, const LatentGeom& g, void* k, void* vt, const float* raw, const float* q,
+                                const int* pos, float* qa, hipStream_t s);
+int latent_slices(int window, int max_seq);
+// o [slice][heads][Dc] (not divided), ml [slice][heads] (max, sum)
+hipError_t launch_latent_decode(int dtype, const LatentGeom& g, const void* k, const void* vt, const float* qa,
+                                const int* pos, int max_seq, float* o, float* ml, hipStream_t s);
+// slices merged, values read out of the latents, gates: y f32 [heads * vdim]
+hipError_t launch_latent_out(int dtype, const LatentGeom& g, const float* o, const float* ml, int slices, const float* raw,
+                             float* y, hipStream_t s);
+
+// ---- mixture of experts ----
+struct MoeGeom {
+  int hidden, Hp, ff, Fp, experts, top;
+  float limit;
+};
+size_t moe_scratch_bytes(int dtype, int M, int experts, int top, int Fp);
+// rows: h T [M][Hp], router logits f32 [logit_parts][M][ldl] -> parts f32 [top][M][Hp]
+hipError_t launch_moe_prefill(int dtype, const MoeGeom& g, const void* h, const float* logits, int logit_parts, int ldl,
+                              const void* gate_up, const void* down, int M, float* parts, void* scratch, hipStream_t s);
+// one token: pro is the norm in front (its x_out must be null), z f32 [top * Fp], sel int [top]; out f32 [Hp]
+bool moe_decode_fits(const MoeGeom& g);
+hipError_t launch_moe_decode(int dtype, const MoeGeom& g, const RowPrologue& pro, const float* logits, const void* gate_up,
+                             const void* down, float* z, int* sel, float* out, hipStream_t s);
 
 // ---- recurrences with a matrix state ----
 // State of a layer: f32 [heads][dv16][D], transposed (a value row's D key dimensions are contiguous); dv16 = vdim
@@ -182,7 +254,7 @@ hipError_t launch_rec_prefill(int dtype, const RecGeom& g, const float* raw, con
 // one token: o f32 [heads * vdim], before norm and gate
 hipError_t launch_rec_decode(const RecGeom& g, const float* raw, const float* conv, float* ring, float* state,
                              const int* pos, float* o, hipStream_t s);
-hipError_t launch_rot_table(float* sin_t, float* cos_t, int max_pos, int dims, float base, hipStream_t s);
+hipError_t launch_rot_table(float* sin_t, float* cos_t, int max_pos, int dims, double base, hipStream_t s);
 hipError_t launch_fill_zero(void* p, size_t bytes, hipStream_t s);  // bytes % 16 == 0
 
 }  // namespace w4

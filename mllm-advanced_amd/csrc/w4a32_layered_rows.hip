@@ -27,15 +27,15 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(const int64_t* __restri
   for (int c = 4 * threadIdx.x; c < ld; c += 1024) store4(dst + c, load4(src + c));
 }
 
-// Layer norm of one row by one wavefront: x + parts -> LDS row s_h (h, zeros past H). The completed residual row goes to
+// Layer norm (or the norm that takes no mean off) of one row by one wavefront: x + scale * parts -> LDS row s_h (h, zeros past H). The completed residual row goes to
 // x_out when that is given. Rows of up to 2048 channels stay in registers on the way.
 __device__ __forceinline__ void wave_layer_norm(const float* __restrict__ x, const float* __restrict__ parts,
                                                 int n_parts, size_t part_stride, float* __restrict__ x_out,
-                                                const float* __restrict__ w, float eps, int H, int ld,
+                                                const float* __restrict__ w, const NormSpec& spec, int H, int ld,
                                                 float* __restrict__ s_h) {
   const int lane = threadIdx.x & 63;
-  const float inv = 1.0f / (float)H;
-  auto add = [](float4& v, const float4& d) { v.x += d.x; v.y += d.y; v.z += d.z; v.w += d.w; };
+  const float inv = 1.0f / (float)H, eps = spec.eps, ps = spec.part_scale;
+  auto add = [ps](float4& v, const float4& d) { v.x += ps * d.x; v.y += ps * d.y; v.z += ps * d.z; v.w += ps * d.w; };
   auto clip = [&](float4& v, int c) {
     if (c + 3 >= H) {
 #pragma unroll
@@ -77,7 +77,7 @@ __device__ __forceinline__ void wave_layer_norm(const float* __restrict__ x, con
       if (x_out && c < ld) store4(x_out + c, v[i]);
       sum += (v[i].x + v[i].y) + (v[i].z + v[i].w);
     }
-    const float mean = wave_sum64(sum) * inv;
+    const float mean = spec.rms ? 0.0f : wave_sum64(sum) * inv;
     float ss = 0.0f;
 #pragma unroll
     for (int i = 0; i < kRegs; ++i) ss += square(v[i], 4 * lane + 256 * i, mean);
@@ -100,7 +100,7 @@ __device__ __forceinline__ void wave_layer_norm(const float* __restrict__ x, con
     store4(s_h + c, v);
     sum += (v.x + v.y) + (v.z + v.w);
   }
-  const float mean = wave_sum64(sum) * inv;
+  const float mean = spec.rms ? 0.0f : wave_sum64(sum) * inv;
   float ss = 0.0f;
   for (int c = 4 * lane; c < ld; c += 256) ss += square(load4(s_h + c), c, mean);  // the elements this lane wrote
   const float rstd = 1.0f / sqrtf(wave_sum64(ss) * inv + eps);
@@ -118,7 +118,7 @@ constexpr int kNcWaves = 8;
 template <int TAPS, typename YT>
 __global__ __launch_bounds__(64 * kNcWaves) void norm_conv_kernel(
     const float* __restrict__ x, const float* __restrict__ parts, int n_parts, float* __restrict__ x_out,
-    const float* __restrict__ norm_w, float eps, const float* __restrict__ conv, float* __restrict__ ring, int M, int H,
+    const float* __restrict__ norm_w, NormSpec spec, const float* __restrict__ conv, float* __restrict__ ring, int M, int H,
     int ld, int pos0, int TR, YT* __restrict__ y) {
   extern __shared__ __align__(16) float s_h[];  // [halo + TR][ld]
   constexpr int halo = TAPS > 0 ? TAPS - 1 : 0, kRing = TAPS > 0 ? TAPS : 1;
@@ -132,7 +132,7 @@ __global__ __launch_bounds__(64 * kNcWaves) void norm_conv_kernel(
     float* dst = s_h + (size_t)r * ld;
     if (t >= 0) {
       wave_layer_norm(x + (size_t)t * ld, parts + (size_t)t * ld, n_parts, (size_t)M * ld,
-                      x_out && r >= halo ? x_out + (size_t)t * ld : nullptr, norm_w, eps, H, ld, dst);
+                      x_out && r >= halo ? x_out + (size_t)t * ld : nullptr, norm_w, spec, H, ld, dst);
     } else {
       const int q = pos0 + t;
       for (int c = 4 * (threadIdx.x & 63); c < ld; c += 256)
@@ -172,7 +172,7 @@ __global__ __launch_bounds__(64 * kNcWaves) void norm_conv_kernel(
     float* row = s_h + (size_t)(halo + t) * ld;
     if (t >= rows) {
       row = s_h + (size_t)wave * ld;
-      wave_layer_norm(x + (size_t)t * ld, parts + (size_t)t * ld, n_parts, (size_t)M * ld, nullptr, norm_w, eps, H, ld,
+      wave_layer_norm(x + (size_t)t * ld, parts + (size_t)t * ld, n_parts, (size_t)M * ld, nullptr, norm_w, spec, H, ld,
                       row);
     }
     float* dst = ring + (size_t)((pos0 + t) % kRing) * ld;
@@ -183,26 +183,45 @@ static_assert(kNcWaves >= W4A32_LAYERED_MAX_TAPS - 1, "a wavefront per row of th
 
 template <typename YT>
 __global__ __launch_bounds__(64) void norm_want_kernel(const float* __restrict__ x, const float* __restrict__ parts,
-                                                       int n_parts, const float* __restrict__ norm_w, float eps,
-                                                       const int* __restrict__ want, int M, int H, int ld,
+                                                       int n_parts, const float* __restrict__ norm_w,
+                                                       NormSpec spec, const int* __restrict__ want, int M, int H, int ld,
                                                        YT* __restrict__ y) {
   extern __shared__ __align__(16) float s_h[];
   const int t = min(max(want[blockIdx.x], 0), M - 1);
-  wave_layer_norm(x + (size_t)t * ld, parts + (size_t)t * ld, n_parts, (size_t)M * ld, nullptr, norm_w, eps, H, ld,
+  wave_layer_norm(x + (size_t)t * ld, parts + (size_t)t * ld, n_parts, (size_t)M * ld, nullptr, norm_w, spec, H, ld,
                   s_h);
   for (int c = 4 * threadIdx.x; c < ld; c += 256) store4(y + (size_t)blockIdx.x * ld + c, load4(s_h + c));
 }
 
 __global__ __launch_bounds__(256) void add_parts_kernel(const float* x, const float* __restrict__ parts,
-                                                        int n_parts, float* out, size_t n) {
+                                                        int n_parts, float scale, float* out, size_t n) {
   const size_t i = 4 * ((size_t)blockIdx.x * 256 + threadIdx.x);
   if (i >= n) return;
   float4 v = load4(x + i);
   for (int p = 0; p < n_parts; ++p) {
     const float4 d = load4(parts + p * n + i);
-    v.x += d.x; v.y += d.y; v.z += d.z; v.w += d.w;
+    v.x += scale * d.x; v.y += scale * d.y; v.z += scale * d.z; v.w += scale * d.w;
   }
   store4(out + i, v);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void loop_rows_kernel(const float* __restrict__ x, const float* __restrict__ parts,
+                                                        int n_parts, float scale, const int64_t* __restrict__ ids,
+                                                        const T* __restrict__ table, int vocab, size_t part_stride,
+                                                        int ld, T* __restrict__ y) {
+  const size_t row = (size_t)blockIdx.x * ld;
+  const int64_t id = ids[blockIdx.x];
+  const T* src = table + (size_t)(id < 0 ? 0 : id >= vocab ? vocab - 1 : id) * ld;
+  for (int c = 4 * threadIdx.x; c < ld; c += 1024) {
+    float4 v = load4(x + row + c);
+    for (int p = 0; p < n_parts; ++p) {
+      const float4 d = load4(parts + p * part_stride + row + c);
+      v.x += scale * d.x; v.y += scale * d.y; v.z += scale * d.z; v.w += scale * d.w;
+    }
+    store4(y + 2 * row + c, v);
+    store4(y + 2 * row + ld + c, load4(src + c));
+  }
 }
 
 template <typename ZT>
@@ -306,10 +325,10 @@ hipError_t launch_fill_zero(void* p, size_t bytes, hipStream_t s) {
   return hipGetLastError();
 }
 
-hipError_t launch_rot_table(float* sin_t, float* cos_t, int max_pos, int dims, float base, hipStream_t s) {
+hipError_t launch_rot_table(float* sin_t, float* cos_t, int max_pos, int dims, double base, hipStream_t s) {
   const size_t n = (size_t)max_pos * (dims / 2);
   hipLaunchKernelGGL(rot_table_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, sin_t, cos_t, max_pos, dims,
-                     (double)base);
+                     base);
   return hipGetLastError();
 }
 
@@ -343,7 +362,7 @@ bool norm_conv_fits(int ld, int taps) { return norm_conv_lds(ld, taps, 1) <= 160
 
 template <int TAPS, typename YT>
 static hipError_t norm_conv_t(const float* x, const float* parts, int n_parts, float* x_out, const float* norm_w,
-                              float eps, const float* conv, float* ring, int M, int H, int ld, int pos0, YT* y,
+                              const NormSpec& spec, const float* conv, float* ring, int M, int H, int ld, int pos0, YT* y,
                               hipStream_t s) {
   const int TR = norm_conv_rows(M, ld, TAPS);
   const size_t lds = norm_conv_lds(ld, TAPS, TR);
@@ -351,21 +370,21 @@ static hipError_t norm_conv_t(const float* x, const float* parts, int n_parts, f
   static LdsLimitOnce raised;
   if (lds > 64 * 1024)
     if (hipError_t e = raised.raise(reinterpret_cast<const void*>(kern), 160 * 1024); e != hipSuccess) return e;
-  hipLaunchKernelGGL(kern, dim3((M + TR - 1) / TR), dim3(64 * kNcWaves), lds, s, x, parts, n_parts, x_out, norm_w, eps,
+  hipLaunchKernelGGL(kern, dim3((M + TR - 1) / TR), dim3(64 * kNcWaves), lds, s, x, parts, n_parts, x_out, norm_w, spec,
                      conv, ring, M, H, ld, pos0, TR, y);
   return hipGetLastError();
 }
 
 hipError_t launch_norm_conv(const float* x, const float* parts, int n_parts, float* x_out, const float* norm_w,
-                            float eps, const float* conv, float* ring, int taps, int M, int H, int ld, int pos0,
+                            const NormSpec& spec, const float* conv, float* ring, int taps, int M, int H, int ld, int pos0,
                             void* y, bool y_bf16, hipStream_t s) {
   if (!norm_conv_fits(ld, taps)) return hipErrorInvalidValue;
   if (n_parts == 0) x_out = nullptr;  // the residual rows stay where they are
 #define W4_NORM_CONV(T)                                                                                            \
   case T:                                                                                                          \
-    return y_bf16 ? norm_conv_t<T>(x, parts, n_parts, x_out, norm_w, eps, conv, ring, M, H, ld, pos0,              \
+    return y_bf16 ? norm_conv_t<T>(x, parts, n_parts, x_out, norm_w, spec, conv, ring, M, H, ld, pos0,              \
                                    static_cast<__bf16*>(y), s)                                                     \
-                  : norm_conv_t<T>(x, parts, n_parts, x_out, norm_w, eps, conv, ring, M, H, ld, pos0,              \
+                  : norm_conv_t<T>(x, parts, n_parts, x_out, norm_w, spec, conv, ring, M, H, ld, pos0,              \
                                    static_cast<float*>(y), s)
   switch (taps) {
     W4_NORM_CONV(0); W4_NORM_CONV(1); W4_NORM_CONV(2); W4_NORM_CONV(3); W4_NORM_CONV(4);
@@ -375,8 +394,8 @@ hipError_t launch_norm_conv(const float* x, const float* parts, int n_parts, flo
 #undef W4_NORM_CONV
 }
 
-hipError_t launch_norm_want(const float* x, const float* parts, int n_parts, const float* norm_w, float eps,
-                            const int* want, int n_want, int M, int H, int ld, void* y, bool y_bf16, hipStream_t s) {
+hipError_t launch_norm_want(const float* x, const float* parts, int n_parts, const float* norm_w,
+                            const NormSpec& spec, const int* want, int n_want, int M, int H, int ld, void* y, bool y_bf16, hipStream_t s) {
   const size_t lds = sizeof(float) * ld;
   if (lds > 160 * 1024) return hipErrorInvalidValue;
   if (y_bf16) {
@@ -385,7 +404,7 @@ hipError_t launch_norm_want(const float* x, const float* parts, int n_parts, con
       if (hipError_t e = raised.raise(reinterpret_cast<const void*>(norm_want_kernel<__bf16>), 160 * 1024);
           e != hipSuccess)
         return e;
-    hipLaunchKernelGGL(norm_want_kernel<__bf16>, dim3(n_want), dim3(64), lds, s, x, parts, n_parts, norm_w, eps, want,
+    hipLaunchKernelGGL(norm_want_kernel<__bf16>, dim3(n_want), dim3(64), lds, s, x, parts, n_parts, norm_w, spec, want,
                        M, H, ld, static_cast<__bf16*>(y));
   } else {
     static LdsLimitOnce raised;
@@ -393,17 +412,30 @@ hipError_t launch_norm_want(const float* x, const float* parts, int n_parts, con
       if (hipError_t e = raised.raise(reinterpret_cast<const void*>(norm_want_kernel<float>), 160 * 1024);
           e != hipSuccess)
         return e;
-    hipLaunchKernelGGL(norm_want_kernel<float>, dim3(n_want), dim3(64), lds, s, x, parts, n_parts, norm_w, eps, want, M,
+    hipLaunchKernelGGL(norm_want_kernel<float>, dim3(n_want), dim3(64), lds, s, x, parts, n_parts, norm_w, spec, want, M,
                        H, ld, static_cast<float*>(y));
   }
   return hipGetLastError();
 }
 
-hipError_t launch_add_parts(const float* x, const float* parts, int n_parts, float* out, int M, int ld,
+hipError_t launch_loop_rows(int dtype, const float* x, const float* parts, int n_parts, float scale, const int64_t* ids,
+                            const void* table, int vocab, int M, int ld, void* y, hipStream_t s) {
+  const size_t stride = (size_t)M * ld;
+  if (dtype == W4A32_LAYERED_BF16) {
+    hipLaunchKernelGGL(loop_rows_kernel<__bf16>, dim3(M), dim3(256), 0, s, x, parts, n_parts, scale, ids,
+                       static_cast<const __bf16*>(table), vocab, stride, ld, static_cast<__bf16*>(y));
+  } else {
+    hipLaunchKernelGGL(loop_rows_kernel<float>, dim3(M), dim3(256), 0, s, x, parts, n_parts, scale, ids,
+                       static_cast<const float*>(table), vocab, stride, ld, static_cast<float*>(y));
+  }
+  return hipGetLastError();
+}
+
+hipError_t launch_add_parts(const float* x, const float* parts, int n_parts, float scale, float* out, int M, int ld,
                             hipStream_t s) {
   const size_t n = (size_t)M * ld;
-  hipLaunchKernelGGL(add_parts_kernel, dim3((unsigned)((n / 4 + 255) / 256)), dim3(256), 0, s, x, parts, n_parts, out,
-                     n);
+  hipLaunchKernelGGL(add_parts_kernel, dim3((unsigned)((n / 4 + 255) / 256)), dim3(256), 0, s, x, parts, n_parts,
+                     scale, out, n);
   return hipGetLastError();
 }
 

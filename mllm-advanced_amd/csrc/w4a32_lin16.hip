@@ -2,125 +2,47 @@
 //
 //   matmul_bf16_kernel   C = A B^T, bf16 operands, f32 accumulation (v_mfma_f32_32x32x16_bf16), for prefill rows.
 //   row_linear_kernel    one decode row through [N][K] weights, read once, with the operator that produces the row
-//                        in front (residual add + layer norm + input convolution, merge of the attention's key
-//                        slices, per-head norm and gate, PolyNorm): HBM-bound, N * K * sizeof(weight) bytes.
+//                        in front (residual add + norm + input convolution, merge of the attention's key slices,
+//                        per-head norm and gate, PolyNorm, none): HBM-bound, N * K * sizeof(weight) bytes.
 //
-// matmul_bf16_kernel: a workgroup of four wavefronts owns a BM x BN tile of C. Tiles of 64 k are brought in through
-// registers (requested one or two tiles ahead) and double-buffered in LDS as rows of 64 + 8 elements: the 144-byte stride
-// puts 16 consecutive rows' 16-byte operands on all 64 banks once. Workgroups are numbered so that one XCD (number
-// mod 8) gets consecutive tiles, rows of C fastest: a band of B stays in that XCD's L2 while all of A passes.
+// The tile of C a workgroup owns and the rows a decode Linear multiplies are in w4a32_mfma_tile.h and w4a32_row_prologue.h.
 #include <algorithm>
 
 #include "w4a32_layered.h"
 #include "w4a32_layered_kernels.h"
+#include "w4a32_mfma_tile.h"
+#include "w4a32_row_prologue.h"
 
 namespace w4 {
 
 namespace {
 
-constexpr int kBK = 64;          // k per LDS tile
-constexpr int kLd = kBK + 8;     // LDS row, elements
-
 template <int BM, int BN, int WM, int WN, typename CT>
 __global__ __launch_bounds__(64 * WM * WN) void matmul_bf16_kernel(const __bf16* __restrict__ a,
                                                                    const __bf16* __restrict__ b, CT* __restrict__ c,
                                                                    int M, int N, int K, int ldc, int mt, int nt) {
-  constexpr int kThreads = 64 * WM * WN;
-  constexpr int FM = BM / WM / 32, FN = BN / WN / 32;           // 32 x 32 blocks of a wavefront
-  constexpr int LA = BM * 8 / kThreads, LB = BN * 8 / kThreads;  // 16-byte pieces a thread brings per tile
+  using Tile = MfmaTile<__bf16, BM, BN, WM, WN>;
+  constexpr int FM = Tile::FM, FN = Tile::FN, kBK = Tile::kBK;
   extern __shared__ __align__(16) uint8_t smem[];
-  __bf16* s_a = reinterpret_cast<__bf16*>(smem);                 // [2][BM][kLd]
-  __bf16* s_b = s_a + 2 * BM * kLd;                              // [2][BN][kLd]
 
   // tile number: consecutive ones on one XCD
-  const int tiles = mt * nt;
-  int t = blockIdx.x;
-  {
-    const int per = tiles / 8, rem = tiles % 8, x = t & 7, i = t >> 3;
-    t = x * per + min(x, rem) + i;  // XCD x holds per (+ 1 for x < rem) tiles
-  }
+  const int t = xcd_tile(blockIdx.x, mt * nt);
   const int m0 = (t % mt) * BM, n0 = (t / mt) * BN;
   // this workgroup's share of the k range, in whole LDS tiles
   const int k_steps = K / kBK;
   const int kb = (int)((long)k_steps * blockIdx.y / gridDim.y) * kBK;
   const int ke = (int)((long)k_steps * (blockIdx.y + 1) / gridDim.y) * kBK;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int wm = (wave / WN) * (BM / WM), wn = (wave % WN) * (BN / WN);
 
-  const __bf16* ga[LA];
-  const __bf16* gb[LB];
+  const __bf16* ga[Tile::LA];
+  const __bf16* gb[Tile::LB];
 #pragma unroll
-  for (int i = 0; i < LA; ++i) {
-    const int r = (tid + kThreads * i) >> 3;
-    ga[i] = a + (size_t)min(m0 + r, M - 1) * K + 8 * (tid & 7);
-  }
+  for (int i = 0; i < Tile::LA; ++i) ga[i] = a + (size_t)min(m0 + Tile::row(i), M - 1) * K + Tile::k();
 #pragma unroll
-  for (int i = 0; i < LB; ++i) {
-    const int r = (tid + kThreads * i) >> 3;
-    gb[i] = b + (size_t)min(n0 + r, N - 1) * K + 8 * (tid & 7);
-  }
-  // two register sets: two tiles in flight
-  u32x4 ra0[LA], rb0[LB], ra1[LA], rb1[LB];
-  auto fetch = [&](int k, u32x4 (&ra)[LA], u32x4 (&rb)[LB]) __attribute__((always_inline)) {
-#pragma unroll
-    for (int i = 0; i < LA; ++i) ra[i] = *reinterpret_cast<const u32x4*>(ga[i] + k);
-#pragma unroll
-    for (int i = 0; i < LB; ++i) rb[i] = *reinterpret_cast<const u32x4*>(gb[i] + k);
-  };
-  __bf16* const sa_w = s_a + (tid >> 3) * kLd + 8 * (tid & 7);
-  __bf16* const sb_w = s_b + (tid >> 3) * kLd + 8 * (tid & 7);
-  auto stash = [&](int buf, const u32x4 (&ra)[LA], const u32x4 (&rb)[LB]) __attribute__((always_inline)) {
-#pragma unroll
-    for (int i = 0; i < LA; ++i) *reinterpret_cast<u32x4*>(sa_w + (buf * BM + kThreads / 8 * i) * kLd) = ra[i];
-#pragma unroll
-    for (int i = 0; i < LB; ++i) *reinterpret_cast<u32x4*>(sb_w + (buf * BN + kThreads / 8 * i) * kLd) = rb[i];
-  };
+  for (int i = 0; i < Tile::LB; ++i) gb[i] = b + (size_t)min(n0 + Tile::row(i), N - 1) * K + Tile::k();
   f32x16 acc[FM][FN];
-#pragma unroll
-  for (int i = 0; i < FM; ++i)
-#pragma unroll
-    for (int j = 0; j < FN; ++j)
-#pragma unroll
-      for (int v = 0; v < 16; ++v) acc[i][j][v] = 0.0f;
-
-  auto products = [&](int buf) __attribute__((always_inline)) {
-    const __bf16* pa = s_a + (size_t)buf * BM * kLd + (wm + (lane & 31)) * kLd + 8 * (lane >> 5);
-    const __bf16* pb = s_b + (size_t)buf * BN * kLd + (wn + (lane & 31)) * kLd + 8 * (lane >> 5);
-#pragma unroll
-    for (int ks = 0; ks < kBK / 16; ++ks) {
-      bf16x8 fa[FM], fb[FN];
-#pragma unroll
-      for (int i = 0; i < FM; ++i) fa[i] = *reinterpret_cast<const bf16x8*>(pa + 32 * i * kLd + 16 * ks);
-#pragma unroll
-      for (int j = 0; j < FN; ++j) fb[j] = *reinterpret_cast<const bf16x8*>(pb + 32 * j * kLd + 16 * ks);
-#pragma unroll
-      for (int i = 0; i < FM; ++i)
-#pragma unroll
-        for (int j = 0; j < FN; ++j)
-          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
-    }
-  };
-
-  // Tile i is stashed from register set i & 1 into LDS buffer i & 1; while it is multiplied, tiles i + 1 and i + 2
-  // are on their way.
-  const int last = ke - kBK;  // a tile past the end is fetched as the last one again and not used
-  fetch(kb, ra0, rb0);
-  fetch(min(kb + kBK, last), ra1, rb1);
-  stash(0, ra0, rb0);
-  fetch(min(kb + 2 * kBK, last), ra0, rb0);
-  __syncthreads();
-  for (int k = kb; k < ke; k += 2 * kBK) {
-    // even tile: LDS buffer 0; the next one sits in register set 1
-    stash(1, ra1, rb1);
-    fetch(min(k + 3 * kBK, last), ra1, rb1);
-    products(0);
-    __syncthreads();
-    if (k + kBK >= ke) break;
-    stash(0, ra0, rb0);
-    fetch(min(k + 4 * kBK, last), ra0, rb0);
-    products(1);
-    __syncthreads();
-  }
+  Tile::run(smem, ga, gb, kb, ke, acc);
 
   c += (size_t)blockIdx.y * M * ldc;
 #pragma unroll
@@ -141,7 +63,7 @@ hipError_t launch_tile(const __bf16* a, const __bf16* b, void* c, int M, int N, 
                        hipStream_t s) {
   const int mt = (M + BM - 1) / BM, nt = (N + BN - 1) / BN;
   const dim3 grid(mt * nt, parts), block(64 * WM * WN);  // parts <= K / kBK: no share is empty
-  constexpr size_t lds = 2 * (BM + BN) * kLd * sizeof(__bf16);
+  constexpr size_t lds = MfmaTile<__bf16, BM, BN, WM, WN>::kLds;
   if (c_bf16) {
     auto kern = matmul_bf16_kernel<BM, BN, WM, WN, __bf16>;
     static LdsLimitOnce raised;
@@ -163,331 +85,6 @@ long tiles_of(int M, int N, int t) { return (long)((M + t - 1) / t) * ((N + t - 
 bool small_tiles(int M, int N, int parts) { return tiles_of(M, N, 128) < (parts > 1 ? 96 : 192); }
 
 // ---------------------------------------------------------------------------------------------
-constexpr int kRowThreads = 512, kRowWaves = kRowThreads / 64;
-
-// Sums over the workgroup of N values per thread, in every thread; s_red holds N * kRowWaves floats.
-template <int N>
-__device__ __forceinline__ void block_totals(float (&v)[N], float* s_red) {
-#pragma unroll
-  for (int i = 0; i < N; ++i) {
-    v[i] = wave_sum64(v[i]);
-    if ((threadIdx.x & 63) == 0) s_red[i * kRowWaves + (threadIdx.x >> 6)] = v[i];
-  }
-  __syncthreads();
-#pragma unroll
-  for (int i = 0; i < N; ++i) {
-    v[i] = 0.0f;
-#pragma unroll
-    for (int w = 0; w < kRowWaves; ++w) v[i] += s_red[i * kRowWaves + w];
-  }
-}
-
-// Mean and 1 / sqrt(variance + eps) of K values, of which each wavefront holds `n` with sum `sum` (this lane's share);
-// `spread(mean)` returns the lane's share of the squared deviations from a mean. One barrier: the wavefronts'
-// means and squared deviations are combined, which loses no digits to the mean's size.
-template <typename Spread>
-__device__ __forceinline__ void block_norm_stats(float sum, float n, float K, float eps, Spread spread, float* s_red,
-                                                 float* mean_out, float* rstd_out) {
-  const float m = n > 0.0f ? wave_sum64(sum) / n : 0.0f;
-  const float d = wave_sum64(spread(m));
-  if ((threadIdx.x & 63) == 0) {
-    const int w = threadIdx.x >> 6;
-    s_red[w] = n;
-    s_red[kRowWaves + w] = m;
-    s_red[2 * kRowWaves + w] = d;
-  }
-  __syncthreads();
-  float mean = 0.0f, dev = 0.0f;
-#pragma unroll
-  for (int w = 0; w < kRowWaves; ++w) mean = __fmaf_rn(s_red[w], s_red[kRowWaves + w], mean);
-  mean /= K;
-#pragma unroll
-  for (int w = 0; w < kRowWaves; ++w) {
-    const float e = s_red[kRowWaves + w] - mean;
-    dev += s_red[2 * kRowWaves + w] + s_red[w] * e * e;
-  }
-  *mean_out = mean;
-  *rstd_out = 1.0f / sqrtf(dev / K + eps);
-}
-
-// The row a decode Linear multiplies, into s_x [Kp] (zeros past K), by 512 threads. Each kind comes in two steps, what it
-// requests from memory and what it makes of that: a CU's loads return in the order they were issued, so the
-// row's inputs are requested in front of the first weights and the arithmetic runs while those arrive. Rows that
-// do not fit one step's registers are read in the second one.
-constexpr int kFastTaps = 4;  // input convolutions up to this length are requested ahead
-
-struct NormRegs {
-  bool fast;
-  int pos;
-  f32x4 x, w, cw[kFastTaps], rg[kFastTaps];
-};
-
-__device__ __forceinline__ f32x4 load_row4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
-__device__ __forceinline__ f32x4 load_row4(const __bf16* p) {
-  const float4 v = load4(p);
-  return f32x4{v.x, v.y, v.z, v.w};
-}
-__device__ __forceinline__ void store_row4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
-
-template <typename WT>
-__device__ __forceinline__ const WT* token_row(const RowPrologue& p, int Kp) {
-  if (!p.token) return nullptr;
-  const int64_t id = *p.token;
-  return static_cast<const WT*>(p.table) + (size_t)(id < 0 ? 0 : id >= p.vocab ? p.vocab - 1 : id) * Kp;
-}
-
-template <typename WT>
-__device__ __forceinline__ f32x4 norm_input(const RowPrologue& p, const WT* trow, int c) {
-  f32x4 v = trow ? load_row4(trow + c) : load_row4(p.x + c);
-  for (int i = 0; i < p.n_parts; ++i) v += load_row4(p.parts + i * p.part_stride + c);
-  return v;
-}
-
-template <typename WT>
-__device__ __forceinline__ void row_norm_request(const RowPrologue& p, int Kp, NormRegs& r) {
-  r.fast = Kp <= 4 * kRowThreads && p.taps <= kFastTaps;
-  r.pos = p.taps > 0 ? *p.pos : 0;
-  if (!r.fast) return;
-  const int c = min(4 * (int)threadIdx.x, Kp - 4);
-  r.x = norm_input(p, token_row<WT>(p, Kp), c);
-  r.w = load_row4(p.norm_w + c);
-#pragma unroll
-  for (int j = 0; j < kFastTaps; ++j) {
-    r.cw[j] = r.rg[j] = f32x4{0, 0, 0, 0};
-    if (j < p.taps) {
-      r.cw[j] = load_row4(p.conv + (size_t)j * Kp + c);
-      const int q = r.pos - p.taps + 1 + j;
-      if (q >= 0 && q < r.pos) r.rg[j] = load_row4(p.ring + (size_t)(q % p.taps) * Kp + c);
-    }
-  }
-}
-
-template <typename WT>
-__device__ __forceinline__ void row_norm(const RowPrologue& p, int Kp, const NormRegs& r, float* s_x, float* s_red) {
-  const bool first_wg = blockIdx.x == 0;
-  const int c0 = 4 * threadIdx.x;
-  float mean, rstd;
-  if (r.fast) {
-    // one vector per thread
-    f32x4 x = r.x;
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (c0 + e >= p.K) x[e] = 0.0f;
-    const int w0 = 4 * ((int)threadIdx.x & ~63);  // the wavefront's columns
-    block_norm_stats((x[0] + x[1]) + (x[2] + x[3]), (float)min(max(p.K - w0, 0), 256), (float)p.K, p.eps,
-                     [&](float m) {
-                       float ss = 0.0f;
-#pragma unroll
-                       for (int e = 0; e < 4; ++e) {
-                         const float d = c0 + e < p.K ? x[e] - m : 0.0f;
-                         ss += d * d;
-                       }
-                       return ss;
-                     },
-                     s_red, &mean, &rstd);
-    if (c0 < Kp) {
-      if (p.x_out && first_wg) store_row4(p.x_out + c0, x);
-      const f32x4 h = (x - mean) * rstd * r.w;
-      if (p.taps > 0 && first_wg) store_row4(p.ring + (size_t)(r.pos % p.taps) * Kp + c0, h);
-      f32x4 y = h;
-#pragma unroll
-      for (int j = 0; j < kFastTaps; ++j) y += r.cw[j] * (j == p.taps - 1 ? h : r.rg[j]);
-      store_row4(s_x + c0, y);
-    }
-    return;
-  }
-  const WT* trow = token_row<WT>(p, Kp);
-  float sum = 0.0f, count = 0.0f;
-  for (int c = c0; c < Kp; c += 4 * kRowThreads) {
-    f32x4 v = norm_input(p, trow, c);
-    count += (float)min(max(p.K - (c & ~255), 0), 256);
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (c + e >= p.K) v[e] = 0.0f;
-    store_row4(s_x + c, v);
-    sum += (v[0] + v[1]) + (v[2] + v[3]);
-  }
-  // (a wavefront whose last columns lie past Kp counts in its first lane's terms: they cover the whole wavefront)
-  block_norm_stats(sum, __shfl(count, 0, 64), (float)p.K, p.eps,
-                   [&](float m) {
-                     float ss = 0.0f;
-                     for (int c = c0; c < Kp; c += 4 * kRowThreads) {
-                       const f32x4 v = load_row4(s_x + c);
-#pragma unroll
-                       for (int e = 0; e < 4; ++e) {
-                         const float d = c + e < p.K ? v[e] - m : 0.0f;
-                         ss += d * d;
-                       }
-                     }
-                     return ss;
-                   },
-                   s_red, &mean, &rstd);
-  for (int c = c0; c < Kp; c += 4 * kRowThreads) {
-    const f32x4 v = load_row4(s_x + c);
-    if (p.x_out && first_wg) store_row4(p.x_out + c, v);
-    const f32x4 h = (v - mean) * rstd * load_row4(p.norm_w + c);
-    if (p.taps > 0 && first_wg) store_row4(p.ring + (size_t)(r.pos % p.taps) * Kp + c, h);
-    f32x4 y = h;
-    for (int j = 0; j < p.taps; ++j) {
-      const int q = r.pos - p.taps + 1 + j;
-      if (q < 0) continue;
-      y += load_row4(p.conv + (size_t)j * Kp + c) * (q == r.pos ? h : load_row4(p.ring + (size_t)(q % p.taps) * Kp + c));
-    }
-    store_row4(s_x + c, y);
-  }
-}
-
-struct MergeRegs {
-  bool fast;
-  int head;
-  f32x4 part[kPoolAttnSlices];
-};
-
-__device__ __forceinline__ void row_merge_request(const RowPrologue& p, int Kp, MergeRegs& r) {
-  r.fast = (p.vdim & 3) == 0 && Kp <= 4 * kRowThreads;
-  if (!r.fast) return;
-  const int c = min(4 * (int)threadIdx.x, p.K - 4);
-  r.head = c / p.vdim;
-  const float* src = p.o + (size_t)r.head * p.dvp + (c - r.head * p.vdim);
-#pragma unroll
-  for (int i = 0; i < kPoolAttnSlices; ++i)
-    r.part[i] = load_row4(src + (size_t)min(i, p.slices - 1) * p.heads * p.dvp);
-}
-
-// s_w: [kPoolAttnSlices][heads], the slices' weights (behind the row)
-__device__ __forceinline__ void row_merge(const RowPrologue& p, int Kp, const MergeRegs& r, float* s_x, float* s_w) {
-  for (int h = threadIdx.x; h < p.heads; h += kRowThreads) {
-    float m[kPoolAttnSlices], l[kPoolAttnSlices], mx = -INFINITY, den = 0.0f;
-#pragma unroll
-    for (int i = 0; i < kPoolAttnSlices; ++i) {
-      const float2 ml = *reinterpret_cast<const float2*>(p.ml + 2 * ((size_t)min(i, p.slices - 1) * p.heads + h));
-      m[i] = i < p.slices ? ml.x : -INFINITY;
-      l[i] = ml.y;
-      mx = fmaxf(mx, m[i]);
-    }
-#pragma unroll
-    for (int i = 0; i < kPoolAttnSlices; ++i) {
-      m[i] = m[i] == -INFINITY ? 0.0f : expf(m[i] - mx);  // an empty slice holds no keys
-      den = __fmaf_rn(m[i], l[i], den);
-    }
-    const float inv = 1.0f / den;  // the token's own key is always seen
-#pragma unroll
-    for (int i = 0; i < kPoolAttnSlices; ++i) s_w[i * p.heads + h] = m[i] * inv;
-  }
-  __syncthreads();
-  if (r.fast) {
-    const int c = 4 * threadIdx.x;
-    f32x4 y = {0, 0, 0, 0};
-#pragma unroll
-    for (int i = 0; i < kPoolAttnSlices; ++i) y += r.part[i] * s_w[i * p.heads + r.head];
-    if (c < Kp) store_row4(s_x + c, c < p.K ? y : f32x4{0, 0, 0, 0});
-    return;
-  }
-  const size_t stride = (size_t)p.heads * p.dvp;
-  for (int c = threadIdx.x; c < Kp; c += kRowThreads) {
-    float y = 0.0f;
-    if (c < p.K) {
-      const int h = c / p.vdim, d = c - h * p.vdim;
-      for (int i = 0; i < p.slices; ++i)
-        y = __fmaf_rn(s_w[i * p.heads + h], p.o[i * stride + (size_t)h * p.dvp + d], y);
-    }
-    s_x[c] = y;
-  }
-}
-
-// a wavefront takes whole heads
-__device__ __forceinline__ void row_gated(const RowPrologue& p, int Kp, float* s_x) {
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  for (int h = wave; h < p.heads; h += kRowWaves) {
-    constexpr int kPer = W4A32_LAYERED_MAX_DIM / 64;
-    float v[kPer], g[kPer], w[kPer], ss = 0.0f;
-#pragma unroll
-    for (int i = 0; i < kPer; ++i) {
-      const int d = lane + 64 * i;
-      v[i] = g[i] = w[i] = 0.0f;
-      if (d < p.vdim) {
-        v[i] = p.o[h * p.vdim + d];
-        g[i] = p.gate[h * p.vdim + d];
-        w[i] = p.head_w ? p.head_w[d] : 1.0f;
-      }
-      ss += v[i] * v[i];
-    }
-    const float r = 1.0f / sqrtf(wave_sum64(ss) / (float)p.vdim + p.eps);
-#pragma unroll
-    for (int i = 0; i < kPer; ++i) {
-      const int d = lane + 64 * i;
-      if (d < p.vdim) s_x[h * p.vdim + d] = v[i] * r * w[i] * silu_f(g[i]);
-    }
-  }
-  for (int c = p.K + threadIdx.x; c < Kp; c += kRowThreads) s_x[c] = 0.0f;
-}
-
-constexpr int kPolyRegs = 5;
-struct PolyRegs {
-  f32x4 z[kPolyRegs];
-};
-
-__device__ __forceinline__ void row_poly_request(const RowPrologue& p, int Kp, PolyRegs& r) {
-#pragma unroll
-  for (int i = 0; i < kPolyRegs; ++i) r.z[i] = load_row4(p.x + min(4 * ((int)threadIdx.x + kRowThreads * i), Kp - 4));
-}
-
-__device__ __forceinline__ void row_poly(const RowPrologue& p, int Kp, const PolyRegs& r, float* s_x, float* s_red) {
-  float t[3] = {0.0f, 0.0f, 0.0f};
-  auto take = [&](int c, f32x4 z) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      if (c + e >= p.K) z[e] = 0.0f;
-      const float q = z[e] * z[e];
-      t[0] += q;
-      t[1] = __fmaf_rn(q, q, t[1]);
-      t[2] = __fmaf_rn(q * q, q, t[2]);
-    }
-    if (c < Kp) store_row4(s_x + c, z);
-  };
-#pragma unroll
-  for (int i = 0; i < kPolyRegs; ++i) take(4 * ((int)threadIdx.x + kRowThreads * i), r.z[i]);
-  for (int c = 4 * ((int)threadIdx.x + kRowThreads * kPolyRegs); c < Kp; c += 4 * kRowThreads) take(c, load_row4(p.x + c));
-  block_totals(t, s_red);
-  const float inv = 1.0f / (float)p.K, e0 = p.act[3];
-  const float r1 = p.act[0] / sqrtf(t[0] * inv + p.eps);
-  const float r2 = p.act[1] / sqrtf(t[1] * inv + p.eps);
-  const float r3 = p.act[2] / sqrtf(t[2] * inv + p.eps);
-  for (int c = 4 * threadIdx.x; c < Kp; c += 4 * kRowThreads) {  // the elements this thread wrote
-    f32x4 z = load_row4(s_x + c);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) z[e] = c + e < p.K ? z[e] * (r1 + z[e] * (r2 + z[e] * r3)) + e0 : 0.0f;
-    store_row4(s_x + c, z);
-  }
-}
-
-// eight consecutive weights as they come from memory
-template <typename WT>
-struct Raw;
-template <>
-struct Raw<__bf16> {
-  uint4 v;
-  __device__ __forceinline__ void load(const __bf16* p) { v = *reinterpret_cast<const uint4*>(p); }
-  __device__ __forceinline__ float get(int e) const {
-    const uint32_t w = e < 2 ? v.x : e < 4 ? v.y : e < 6 ? v.z : v.w;
-    return __uint_as_float(e & 1 ? w & 0xFFFF0000u : w << 16);
-  }
-};
-template <>
-struct Raw<float> {
-  float4 a, b;
-  __device__ __forceinline__ void load(const float* p) {
-    a = load4(p);
-    b = load4(p + 4);
-  }
-  __device__ __forceinline__ float get(int e) const {
-    const float f[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
-    return f[e];
-  }
-};
-
-// R rows of W at a time per wavefront, lane l multiplies k = 512 i + 8 l .. + 7; U steps of i are in flight while the
-// previous U are multiplied.
 template <typename WT, int kKind, int R, int U>
 __global__ __launch_bounds__(kRowThreads) void row_linear_kernel(const RowPrologue p, const WT* __restrict__ w, int N,
                                                                  int Kp, float* __restrict__ y,
@@ -498,97 +95,30 @@ __global__ __launch_bounds__(kRowThreads) void row_linear_kernel(const RowProlog
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int gw = (int)blockIdx.x * kRowWaves + wave, nw = (int)gridDim.x * kRowWaves;
   const int groups = (N + R - 1) / R;
-  const int steps = (Kp + 511) / 512, batches = (steps + U - 1) / U;
-
-  auto fetch = [&](int g, int bt, Raw<WT> (&raw)[R][U]) {
-#pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const WT* row = w + (size_t)min(g * R + r, N - 1) * Kp;
-#pragma unroll
-      for (int u = 0; u < U; ++u) {
-        const int k = 512 * (bt * U + u) + 8 * lane;
-        raw[r][u].load(row + (k < Kp ? k : 0));
-      }
-    }
-  };
+  auto ptr = [&](int g, int r, int k) { return w + (size_t)min(g * R + r, N - 1) * Kp + k; };
   Raw<WT> cur[R][U];
-  auto first_weights = [&] {
+  row_prologue<WT, kKind>(p, Kp, s_x, s_red, [&] {
     __builtin_amdgcn_sched_barrier(0);
-    if (gw < groups) fetch(gw, 0, cur);
+    if (gw < groups) fetch_rows<WT, R, U>(cur, gw, 0, Kp, ptr);
     __builtin_amdgcn_sched_barrier(0);
-  };
-  if constexpr (kKind == kRowNorm) {
-    NormRegs regs;
-    row_norm_request<WT>(p, Kp, regs);
-    first_weights();
-    row_norm<WT>(p, Kp, regs, s_x, s_red);
-  }
-  if constexpr (kKind == kRowMerge) {
-    MergeRegs regs;
-    row_merge_request(p, Kp, regs);
-    first_weights();
-    row_merge(p, Kp, regs, s_x, s_x + Kp);
-  }
-  if constexpr (kKind == kRowGated) {
-    first_weights();
-    row_gated(p, Kp, s_x);
-  }
-  if constexpr (kKind == kRowPoly) {
-    PolyRegs regs;
-    row_poly_request(p, Kp, regs);
-    first_weights();
-    row_poly(p, Kp, regs, s_x, s_red);
-  }
+  });
   __syncthreads();
 
   float best_v = -INFINITY;
   int best_n = 0x7fffffff;
-  for (int g = gw; g < groups; g += nw) {
-    float acc[R];
-#pragma unroll
-    for (int r = 0; r < R; ++r) acc[r] = 0.0f;
-    for (int bt = 0; bt < batches; ++bt) {
-      Raw<WT> nxt[R][U];
-      const bool last = bt + 1 == batches;
-      const int gn = last ? g + nw : g;
-      if (gn < groups) {
-        fetch(gn, last ? 0 : bt + 1, nxt);
-      } else {
-#pragma unroll
-        for (int r = 0; r < R; ++r)
-#pragma unroll
-          for (int u = 0; u < U; ++u) nxt[r][u] = cur[r][u];
-      }
-#pragma unroll
-      for (int u = 0; u < U; ++u) {
-        const int k = 512 * (bt * U + u) + 8 * lane;
-        if (k < Kp) {
-          const float4 x0 = load4(s_x + k), x1 = load4(s_x + k + 4);
-          const float xs[8] = {x0.x, x0.y, x0.z, x0.w, x1.x, x1.y, x1.z, x1.w};
-#pragma unroll
-          for (int r = 0; r < R; ++r)
-#pragma unroll
-            for (int e = 0; e < 8; ++e) acc[r] = __fmaf_rn(cur[r][u].get(e), xs[e], acc[r]);
-        }
-      }
-#pragma unroll
-      for (int r = 0; r < R; ++r)
-#pragma unroll
-        for (int u = 0; u < U; ++u) cur[r][u] = nxt[r][u];
-    }
+  stream_rows<WT, R, U>(cur, gw, nw, groups, Kp, s_x, ptr, [&](int g, const float (&t)[R]) {
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const float t = wave_sum64(acc[r]);
       const int n = g * R + r;
       if (n < N) {
-        if (lane == 0) y[n] = t;
-        if (t > best_v || (t == best_v && n < best_n)) {
-          best_v = t;
+        if (lane == 0) y[n] = t[r];
+        if (t[r] > best_v || (t[r] == best_v && n < best_n)) {
+          best_v = t[r];
           best_n = n;
         }
       }
     }
-  }
+  });
   if (amax_val && lane == 0) {
     amax_val[gw] = best_v;
     amax_idx[gw] = best_n;
@@ -636,6 +166,8 @@ hipError_t launch_row_t(int kind, const RowPrologue& p, const void* w, int N, in
     case kRowMerge: return launch_row_k<WT, kRowMerge>(p, w, N, Kp, y, av, ai, s);
     case kRowGated: return launch_row_k<WT, kRowGated>(p, w, N, Kp, y, av, ai, s);
     case kRowPoly: return launch_row_k<WT, kRowPoly>(p, w, N, Kp, y, av, ai, s);
+    case kRowPlain: return launch_row_k<WT, kRowPlain>(p, w, N, Kp, y, av, ai, s);
+    case kRowLoop: return launch_row_k<WT, kRowLoop>(p, w, N, Kp, y, av, ai, s);
     default: return hipErrorInvalidValue;
   }
 }
@@ -652,7 +184,7 @@ int matmul_bf16_parts(int M, int N, int K) {
 
 hipError_t launch_matmul_bf16(const void* a, const void* b, void* c, int M, int N, int K, int ldc, bool c_bf16,
                               int parts, hipStream_t s) {
-  if (K % kBK != 0 || parts < 1 || parts > K / kBK || (parts > 1 && c_bf16)) return hipErrorInvalidValue;
+  if (K % kPad != 0 || parts < 1 || parts > K / kPad || (parts > 1 && c_bf16)) return hipErrorInvalidValue;
   const __bf16* pa = static_cast<const __bf16*>(a);
   const __bf16* pb = static_cast<const __bf16*>(b);
   if (small_tiles(M, N, parts)) return launch_tile<64, 64, 2, 2>(pa, pb, c, M, N, K, ldc, c_bf16, parts, s);

@@ -21,6 +21,7 @@
 //                         keys per workgroup; the slices are merged by the Linear that follows
 #include <algorithm>
 
+#include "w4a32_attn_blocks.h"
 #include "w4a32_layered.h"
 #include "w4a32_layered_kernels.h"
 
@@ -28,32 +29,21 @@ namespace w4 {
 
 namespace {
 
-__device__ __forceinline__ int pooled_visible(int p, int window, int pool) {
-  const int before = p - window + 1;  // tokens that lie before the window
-  return before > 0 ? before / pool : 0;
-}
-
-// element (entry, dim) of a kv head's keys / values
-__device__ __forceinline__ size_t k_at(int entry, int d, int D) {
-  return (size_t)(entry >> 5) * (32 * D) + (size_t)((d >> 3) * 32 + (entry & 31)) * 8 + (d & 7);
-}
-__device__ __forceinline__ int v_pos(int o) { return (o & 16) + 8 * ((o >> 2) & 1) + 4 * ((o >> 3) & 1) + (o & 3); }
-__device__ __forceinline__ size_t v_at(int entry, int d, int D) {
-  return (size_t)(entry >> 5) * (32 * D) + (size_t)d * 32 + v_pos(entry & 31);
-}
-
 // ---------------------------------------------------------------------------------------------
 constexpr int kQkvTok = 8;
 
 // One thread per channel and block of tokens. Blocks are aligned to eight absolute positions so that a value
 // channel's eight tokens are one store; the first block also takes the partial one in front of it (so no other
 // block's convolution reaches the ring, which this one rewrites at its end).
-template <typename T, int TAPS>
+// ROT: no convolution, q and k are rotated; with `tied` the values are the keys before that.
+template <typename T, int TAPS, bool ROT>
 __global__ __launch_bounds__(256) void attn_qkv_kernel(const float* __restrict__ raw, int ldr,
                                                        const float* __restrict__ conv, float* __restrict__ ring,
                                                        int ldc, T* __restrict__ q, T* __restrict__ kc,
                                                        T* __restrict__ vt, int heads, int kv_heads, int dim, int vdim,
-                                                       int D, int cap, int channels, int M, int pos0) {
+                                                       int D, int cap, int channels, int M, int pos0, int tied,
+                                                       int rot, const float* __restrict__ sin_t,
+                                                       const float* __restrict__ cos_t) {
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= channels) return;
   const int first = 2 * kQkvTok - (pos0 & (kQkvTok - 1));  // end of block 0
@@ -72,13 +62,24 @@ __global__ __launch_bounds__(256) void attn_qkv_kernel(const float* __restrict__
   const int cc = kind == 0 ? c : kind == 1 ? c - nq : c - nq - nk, hd = kind == 2 ? vdim : dim;
   const int head = cc / hd, d = cc - head * hd;
   T* dst = kind == 0 ? q + (size_t)head * D + d : (kind == 1 ? kc : vt) + (size_t)head * cap * D;
+  const bool turn = ROT && kind < 2 && d < rot, store_v = kind == 2 || (ROT && tied && kind == 1);
+  const int partner = turn ? c + rot_partner(d, rot) - d : c;
+  T* dst_v = vt + (size_t)head * cap * D;
   for (int tb = t0; tb < te;) {
     // up to the next multiple of eight positions
     const int n = min(te - tb, kQkvTok - ((pos0 + tb) & (kQkvTok - 1)));
-    T out[kQkvTok];
+    T out[kQkvTok], turned[kQkvTok];  // as projected (and convolved), and rotated
 #pragma unroll
     for (int i = 0; i < kQkvTok; ++i) {
       if (i >= n) break;
+      if constexpr (ROT) {
+        const float x = raw[(size_t)(tb + i) * ldr + c];
+        out[i] = (T)x;
+        turned[i] = turn ? (T)rotated(x, raw[(size_t)(tb + i) * ldr + partner], d, rot, (size_t)(pos0 + tb + i), sin_t,
+                                      cos_t)
+                         : out[i];
+        continue;
+      }
       win[0] = raw[(size_t)(tb + i) * ldr + c];
       float acc = 0.0f;
 #pragma unroll
@@ -88,21 +89,27 @@ __global__ __launch_bounds__(256) void attn_qkv_kernel(const float* __restrict__
       out[i] = (T)acc;
     }
     const int p = pos0 + tb;
-    if (kind == 2 && n == kQkvTok) {  // eight values of a dimension: two runs of four
+    if (store_v && n == kQkvTok) {  // eight values of a dimension: two runs of four
       struct alignas(sizeof(T) * 4) Four { T e[4]; } lo, hi;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         lo.e[i] = out[i];
         hi.e[i] = out[4 + i];
       }
-      *reinterpret_cast<Four*>(dst + v_at(p, d, D)) = lo;
-      *reinterpret_cast<Four*>(dst + v_at(p + 4, d, D)) = hi;
-    } else {
+      *reinterpret_cast<Four*>(dst_v + v_at(p, d, D)) = lo;
+      *reinterpret_cast<Four*>(dst_v + v_at(p + 4, d, D)) = hi;
+    } else if (store_v) {
+#pragma unroll
+      for (int i = 0; i < kQkvTok; ++i)
+        if (i < n) dst_v[v_at(p + i, d, D)] = out[i];
+    }
+    if (kind < 2) {
 #pragma unroll
       for (int i = 0; i < kQkvTok; ++i) {
         if (i >= n) break;
-        if (kind == 0) dst[(size_t)(tb + i) * heads * D] = out[i];
-        else dst[kind == 1 ? k_at(p + i, d, D) : v_at(p + i, d, D)] = out[i];
+        const T y = ROT ? turned[i] : out[i];
+        if (kind == 0) dst[(size_t)(tb + i) * heads * D] = y;
+        else dst[k_at(p + i, d, D)] = y;
       }
     }
     tb += n;
@@ -131,25 +138,39 @@ __global__ __launch_bounds__(256) void attn_pool_kernel(const T* __restrict__ kc
 }
 
 // ---------------------------------------------------------------------------------------------
-__device__ __forceinline__ f32x16 mfma_bf16(bf16x8 a, bf16x8 b, f32x16 c) {
-  return __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, 0, 0, 0);
-}
-
 constexpr int kMfmaWaves = 4;
+
+// what not every design's attention has
+struct PrefillExtra {
+  const float* sinks;      // [heads], or null
+  const float* gate;       // [M][ldg], a column per head, or null
+  int ldg;
+  int qld, qstride;        // elements between rows and between heads of q
+  int blk0;                // first block that the key and value buffers hold
+  // second part of the keys (KR > 0)
+  const void* kr;
+  size_t kr_block;         // elements between blocks
+  int rot_part, rot_dims;
+  const float *sin_t, *cos_t;
+};
 
 // Workgroup = (head, 32 queries); its wavefronts take the blocks of 32 pooled entries and of 32 tokens round-robin and
 // merge through LDS. S^T = K Q^T: A = keys (lane: key l % 32, dims 16 s + 8 (l / 32) ..), B = queries from LDS.
 // O^T += V^T P^T: A = values (lane: dim 32 c + l % 32, keys in the order the first product's registers have:
 // k-step ks, element e holds key 16 ks + 8 (e / 4) + 4 (l / 32) + e % 4), B = the softmaxed registers.
-template <int D>
+//
+// KR > 0: keys have a second part of 16 KR dimensions, rotated and shared by all heads (latent attention; its first parts
+// and values come expanded, blocks from `blk0` on); q is then as projected, [M][qld] with qstride per head, and its second
+// part is rotated here.
+template <int D, int KR>
 __global__ __launch_bounds__(64 * kMfmaWaves) void attn_mfma_kernel(
     const __bf16* __restrict__ q, const __bf16* __restrict__ kc, const __bf16* __restrict__ vt,
     const __bf16* __restrict__ kp, const __bf16* __restrict__ vpt, __bf16* __restrict__ out, int ldo, int M, int heads,
-    int kv_heads, int dim, int vdim, int cap, int capp, int window, int pool, int pos0, float scale) {
+    int kv_heads, int dim, int vdim, int cap, int capp, int window, int pool, int pos0, float scale, const PrefillExtra x) {
   constexpr int KS = D / 16, C = D / 32, R = 16 * C + 2;  // R: floats a lane hands over in the merge
   extern __shared__ __align__(16) uint8_t smem[];
-  bf16x8* s_q = reinterpret_cast<bf16x8*>(smem);                              // [KS][64 lanes]
-  float* s_merge = reinterpret_cast<float*>(smem + KS * 64 * 16);              // [waves - 1][R][64]
+  bf16x8* s_q = reinterpret_cast<bf16x8*>(smem);                              // [KS + KR][64 lanes]
+  float* s_merge = reinterpret_cast<float*>(smem + (KS + KR) * 64 * 16);       // [waves - 1][R][64]
   const int h = blockIdx.x, g = h / (heads / kv_heads);
   // the later query blocks see more keys (until the window is full): they start first
   const int qb = (int)gridDim.y - 1 - (int)blockIdx.y;
@@ -167,18 +188,41 @@ __global__ __launch_bounds__(64 * kMfmaWaves) void attn_mfma_kernel(
 
   for (int it = threadIdx.x; it < KS * 64; it += 64 * kMfmaWaves) {
     const int s = it >> 6, l = it & 63, d0 = 16 * s + 8 * (l >> 5);
-    bf16x8 v = *reinterpret_cast<const bf16x8*>(q + ((size_t)min(32 * qb + (l & 31), M - 1) * heads + h) * D + d0);
+    const __bf16* src = q + (size_t)min(32 * qb + (l & 31), M - 1) * x.qld + (size_t)h * x.qstride + d0;
+    bf16x8 v;
+    if (KR == 0 || ((x.qstride & 7) == 0 && d0 + 8 <= dim)) {
+      v = *reinterpret_cast<const bf16x8*>(src);
 #pragma unroll
-    for (int e = 0; e < 8; ++e)
-      if (d0 + e >= dim) v[e] = (__bf16)0.0f;
+      for (int e = 0; e < 8; ++e)
+        if (d0 + e >= dim) v[e] = (__bf16)0.0f;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = d0 + e < dim ? src[e] : (__bf16)0.0f;
+    }
     s_q[it] = v;
+  }
+  if constexpr (KR > 0) {
+    for (int it = threadIdx.x; it < KR * 64; it += 64 * kMfmaWaves) {
+      const int s = it >> 6, l = it & 63, d0 = 16 * s + 8 * (l >> 5), m = min(32 * qb + (l & 31), M - 1);
+      const __bf16* src = q + (size_t)m * x.qld + (size_t)h * x.qstride + dim;
+      bf16x8 v;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int d = d0 + e;
+        float y = d < x.rot_part ? (float)src[d] : 0.0f;
+        if (d < x.rot_dims)
+          y = rotated(y, (float)src[rot_partner(d, x.rot_dims)], d, x.rot_dims, (size_t)(pos0 + m), x.sin_t, x.cos_t);
+        v[e] = (__bf16)y;
+      }
+      s_q[KS * 64 + it] = v;
+    }
   }
   __syncthreads();
 
   constexpr int kBlk = 32 * D;  // elements of a block
-  const __bf16* kt = kc + (size_t)g * cap * D + (size_t)tok_first * kBlk + 8 * lane;
+  const __bf16* kt = kc + (size_t)g * cap * D + (size_t)(tok_first - x.blk0) * kBlk + 8 * lane;
   const __bf16* kpt = kp + (size_t)g * capp * D + 8 * lane;
-  const __bf16* vtt = vt + (size_t)g * cap * D + (size_t)tok_first * kBlk + 32 * j + 8 * hh;
+  const __bf16* vtt = vt + (size_t)g * cap * D + (size_t)(tok_first - x.blk0) * kBlk + 32 * j + 8 * hh;
   const __bf16* vptt = vpt + (size_t)g * capp * D + 32 * j + 8 * hh;
 
   f32x16 o[C];
@@ -187,12 +231,21 @@ __global__ __launch_bounds__(64 * kMfmaWaves) void attn_mfma_kernel(
 #pragma unroll
     for (int v = 0; v < 16; ++v) o[c][v] = 0.0f;
   float run_max = -INFINITY, run_sum = 0.0f;
+  if (x.sinks && wave == 0) {  // a term of the denominator without a value
+    run_max = x.sinks[h];
+    run_sum = 1.0f;
+  }
 
-  bf16x8 kop[KS];
+  bf16x8 kop[KS], krop[KR > 0 ? KR : 1];
   auto load_k = [&](int b) {
     const __bf16* src = b < pool_blocks ? kpt + (size_t)b * kBlk : kt + (size_t)(b - pool_blocks) * kBlk;
 #pragma unroll
     for (int s = 0; s < KS; ++s) kop[s] = *reinterpret_cast<const bf16x8*>(src + 512 * s);
+    if constexpr (KR > 0) {
+      const __bf16* rsrc = static_cast<const __bf16*>(x.kr) + (size_t)(tok_first + b - pool_blocks) * x.kr_block + 8 * lane;
+#pragma unroll
+      for (int s = 0; s < KR; ++s) krop[s] = *reinterpret_cast<const bf16x8*>(rsrc + 512 * s);
+    }
   };
   if (wave < blocks) load_k(wave);
   for (int b = wave; b < blocks; b += kMfmaWaves) {
@@ -213,6 +266,13 @@ __global__ __launch_bounds__(64 * kMfmaWaves) void attn_mfma_kernel(
     for (int s = 0; s < KS; s += 2) {  // two accumulators take turns
       st = mfma_bf16(kop[s], s_q[s * 64 + lane], st);
       st1 = mfma_bf16(kop[s + 1], s_q[(s + 1) * 64 + lane], st1);
+    }
+    if constexpr (KR > 0) {
+#pragma unroll
+      for (int s = 0; s < KR; ++s) {
+        if (s & 1) st1 = mfma_bf16(krop[s], s_q[(KS + s) * 64 + lane], st1);
+        else st = mfma_bf16(krop[s], s_q[(KS + s) * 64 + lane], st);
+      }
     }
     if (b + kMfmaWaves < blocks) load_k(b + kMfmaWaves);
     // the range of this block's keys that the lane's query sees
@@ -301,7 +361,8 @@ __global__ __launch_bounds__(64 * kMfmaWaves) void attn_mfma_kernel(
       for (int v = 0; v < 16; ++v) o[c][v] += src[(16 * c + v) * 64] * wt;
   }
   if (32 * qb + j >= M) return;
-  const float inv = 1.0f / total;  // every query sees its own key
+  float inv = 1.0f / total;  // every query sees its own key
+  if (x.gate) inv *= sigmoid_f(x.gate[(size_t)(32 * qb + j) * x.ldg + h]);
   __bf16* row = out + (size_t)(32 * qb + j) * ldo;
 #pragma unroll
   for (int c = 0; c < C; ++c)
@@ -332,22 +393,38 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const T* __restrict__ q, 
                                                        const T* __restrict__ vt, const T* __restrict__ kp,
                                                        const T* __restrict__ vpt, T* __restrict__ out, int ldo,
                                                        int heads, int kv_heads, int dim, int vdim, int D, int cap,
-                                                       int capp, int window, int pool, int pos0, float scale) {
-  __shared__ float s_q[W4A32_LAYERED_MAX_DIM], s_p[64];
+                                                       int capp, int window, int pool, int pos0, float scale,
+                                                       const PrefillExtra x) {
+  __shared__ float s_q[W4A32_LAYERED_MAX_DIM + W4A32_LAYERED_MAX_ROT_PART], s_p[64];
   const int h = blockIdx.x, m = blockIdx.y, lane = threadIdx.x, g = h / (heads / kv_heads);
   const int p = pos0 + m;
-  for (int d = lane; d < dim; d += 64) s_q[d] = (float)q[((size_t)m * heads + h) * D + d];
+  const T* qrow = q + (size_t)m * x.qld + (size_t)h * x.qstride;
+  for (int d = lane; d < dim; d += 64) s_q[d] = (float)qrow[d];
+  for (int d = lane; d < x.rot_part; d += 64) {
+    const T* src = qrow + dim;
+    float y = (float)src[d];
+    if (d < x.rot_dims) y = rotated(y, (float)src[rot_partner(d, x.rot_dims)], d, x.rot_dims, (size_t)p, x.sin_t, x.cos_t);
+    s_q[dim + d] = y;
+  }
   constexpr int kPer = W4A32_LAYERED_MAX_DIM / 64;
   float acc[kPer] = {0};
   float run_max = -INFINITY, run_sum = 0.0f;
+  if (x.sinks) {
+    run_max = x.sinks[h];
+    run_sum = 1.0f;
+  }
   __syncthreads();
-  auto segment = [&](const T* keys, const T* vals, int lo, int hi) {  // entries lo .. hi - 1
+  // entries lo .. hi - 1; the buffers start at block blk0
+  auto segment = [&](const T* keys, const T* vals, int lo, int hi, int blk0) {
+    const int off = 32 * blk0;
     for (int b = lo; b < hi; b += 64) {
       const int n = min(64, hi - b);
       float s = -INFINITY;
       if (lane < n) {
         s = 0.0f;
-        for (int d = 0; d < dim; ++d) s = __fmaf_rn(s_q[d], (float)keys[k_at(b + lane, d, D)], s);
+        for (int d = 0; d < dim; ++d) s = __fmaf_rn(s_q[d], (float)keys[k_at(b + lane - off, d, D)], s);
+        const T* kr = static_cast<const T*>(x.kr) + (size_t)((b + lane) >> 5) * x.kr_block;
+        for (int d = 0; d < x.rot_part; ++d) s = __fmaf_rn(s_q[dim + d], (float)kr[k_at((b + lane) & 31, d, 0)], s);
         s *= scale;
       }
       float mx = s;
@@ -366,18 +443,19 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const T* __restrict__ q, 
         const int d = lane + 64 * i;
         if (d >= vdim) break;
         float a = acc[i] * corr;
-        for (int k = 0; k < n; ++k) a = __fmaf_rn(s_p[k], (float)vals[v_at(b + k, d, D)], a);
+        for (int k = 0; k < n; ++k) a = __fmaf_rn(s_p[k], (float)vals[v_at(b + k - off, d, D)], a);
         acc[i] = a;
       }
     }
   };
-  segment(kp + (size_t)g * capp * D, vpt + (size_t)g * capp * D, 0, pooled_visible(p, window, pool));
-  segment(kc + (size_t)g * cap * D, vt + (size_t)g * cap * D, max(0, p - window + 1), p + 1);
+  segment(kp + (size_t)g * capp * D, vpt + (size_t)g * capp * D, 0, pooled_visible(p, window, pool), 0);
+  segment(kc + (size_t)g * cap * D, vt + (size_t)g * cap * D, max(0, p - window + 1), p + 1, x.blk0);
+  const float gate = x.gate ? sigmoid_f(x.gate[(size_t)m * x.ldg + h]) : 1.0f;
   T* row = out + (size_t)m * ldo;
 #pragma unroll
   for (int i = 0; i < kPer; ++i) {
     const int d = lane + 64 * i;
-    if (d < vdim) row[h * vdim + d] = (T)(acc[i] / run_sum);
+    if (d < vdim) row[h * vdim + d] = (T)(acc[i] / run_sum * gate);
   }
   if (h == heads - 1)
     for (int c = heads * vdim + lane; c < ldo; c += 64) row[c] = (T)0.0f;
@@ -386,37 +464,6 @@ __global__ __launch_bounds__(64) void attn_rows_kernel(const T* __restrict__ q, 
 // ---------------------------------------------------------------------------------------------
 constexpr int kDecThreads = 512, kDecWaves = kDecThreads / 64;
 constexpr int kDecTile = 32 * kDecWaves;  // entries a workgroup scores at a time: a block per wavefront
-
-// eight consecutive elements as they come from memory, and as f32
-template <typename T>
-struct Eight;
-template <>
-struct Eight<__bf16> {
-  u32x4 v;
-  __device__ __forceinline__ void load(const __bf16* p) { v = *reinterpret_cast<const u32x4*>(p); }
-  __device__ __forceinline__ float get(int e) const {
-    return __uint_as_float(e & 1 ? v[e >> 1] & 0xFFFF0000u : v[e >> 1] << 16);
-  }
-  __device__ __forceinline__ void set(float4 a, float4 b) {  // values that are bf16 already
-    v[0] = (__float_as_uint(a.x) >> 16) | (__float_as_uint(a.y) & 0xFFFF0000u);
-    v[1] = (__float_as_uint(a.z) >> 16) | (__float_as_uint(a.w) & 0xFFFF0000u);
-    v[2] = (__float_as_uint(b.x) >> 16) | (__float_as_uint(b.y) & 0xFFFF0000u);
-    v[3] = (__float_as_uint(b.z) >> 16) | (__float_as_uint(b.w) & 0xFFFF0000u);
-  }
-};
-template <>
-struct Eight<float> {
-  f32x4 a, b;
-  __device__ __forceinline__ void load(const float* p) {
-    a = *reinterpret_cast<const f32x4*>(p);
-    b = *reinterpret_cast<const f32x4*>(p + 4);
-  }
-  __device__ __forceinline__ float get(int e) const { return e < 4 ? a[e] : b[e - 4]; }
-  __device__ __forceinline__ void set(float4 x, float4 y) {
-    a = f32x4{x.x, x.y, x.z, x.w};
-    b = f32x4{y.x, y.y, y.z, y.w};
-  }
-};
 
 // grid (slices, kv heads). The blocks of 32 entries that hold visible ones (pooled first, then the window) are dealt to
 // the slices in equal runs; a wavefront scores a block, lane (hh, j) half of the dimensions of entry j. Leaves
@@ -427,7 +474,8 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
     const float* __restrict__ raw, const float* __restrict__ conv, float* __restrict__ ring, int ldc,
     T* __restrict__ kc, T* __restrict__ vt, T* __restrict__ kp, T* __restrict__ vpt, float* __restrict__ o,
     float* __restrict__ ml, const int* __restrict__ d_pos, int max_seq, int heads, int kv_heads, int dim, int vdim,
-    int cap, int capp, int window, int pool, float scale, int taps, int own_kv, int make_pool) {
+    int cap, int capp, int window, int pool, float scale, int taps, int own_kv, int make_pool, int tied, int rot,
+    const float* __restrict__ sin_t, const float* __restrict__ cos_t, const float* __restrict__ sinks) {
   constexpr int NC = D / 16;              // 8-dimension pieces of a lane
   constexpr int kGroups = kDecThreads / D;  // groups of threads that sum values, a thread per dimension
   extern __shared__ __align__(16) float sm[];
@@ -467,7 +515,7 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
   auto channel = [&](int it) {
     const int r = it / D, d = it - r * D;
     if (it >= items || d >= (r <= rep ? dim : vdim)) return -1;
-    return r < rep ? (g * rep + r) * dim + d : r == rep ? nq + g * dim + d : nq + nk + g * vdim + d;
+    return r < rep ? (g * rep + r) * dim + d : r == rep || tied ? nq + g * dim + d : nq + nk + g * vdim + d;
   };
   constexpr int kAhead = 2, kFastTaps = 4;
   const bool ahead = taps > 0 && taps <= kFastTaps;
@@ -506,6 +554,7 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
     if (c >= 0) {
       const int r = it / D, d = it - r * D;
       if (taps > 0 && slice == 0) ring[(size_t)(p % taps) * ldc + c] = x;
+      if (d < rot && r <= rep) y = rotated(x, raw[c + rot_partner(d, rot) - d], d, rot, (size_t)p, sin_t, cos_t);
       y = (float)(T)y;
       if (slice == 0) {
         if (r == rep) kb[k_at(p, d, D)] = (T)y;
@@ -533,8 +582,9 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
   }
   for (int it = tid; it < rep * D; it += kDecThreads) s_o[it] = 0.0f;
   for (int r = tid; r < rep; r += kDecThreads) {
-    s_m[3 * r] = -INFINITY;
-    s_m[3 * r + 1] = 0.0f;
+    const bool sink = sinks && slice == 0;  // a term of the denominator without a value
+    s_m[3 * r] = sink ? sinks[g * rep + r] : -INFINITY;
+    s_m[3 * r + 1] = sink ? 1.0f : 0.0f;
   }
   __syncthreads();
 
@@ -686,15 +736,22 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
 template <typename T>
 hipError_t qkv_t(const AttnGeom& g, const AttnMem& m, const float* raw, int ldr, const float* conv, void* q, int M,
                  int pos0, hipStream_t s) {
-  const int channels = g.heads * g.dim + (g.own_kv ? g.kv_heads * (g.dim + g.vdim) : 0);
+  const int channels = g.heads * g.dim + (g.own_kv ? g.kv_heads * (g.dim + (g.tied ? 0 : g.vdim)) : 0);
   const int first = 2 * kQkvTok - (pos0 & (kQkvTok - 1));
   const int blocks = M <= first ? 1 : 1 + (M - first + kQkvTok - 1) / kQkvTok;
   const dim3 grid((channels + 255) / 256, blocks);
+  if (g.rot_dims > 0 || g.tied) {
+    if (g.taps > 0) return hipErrorInvalidValue;
+    hipLaunchKernelGGL((attn_qkv_kernel<T, 1, true>), grid, dim3(256), 0, s, raw, ldr, nullptr, nullptr, 0,
+                       static_cast<T*>(q), static_cast<T*>(m.k), static_cast<T*>(m.vt), g.heads, g.kv_heads, g.dim, g.vdim,
+                       g.D, g.cap, channels, M, pos0, (int)g.tied, g.rot_dims, g.sin_t, g.cos_t);
+    return hipGetLastError();
+  }
 #define W4_QKV(TP)                                                                                                \
   case TP:                                                                                                        \
-    hipLaunchKernelGGL((attn_qkv_kernel<T, TP>), grid, dim3(256), 0, s, raw, ldr, conv, m.ring, g.ldc,            \
+    hipLaunchKernelGGL((attn_qkv_kernel<T, TP, false>), grid, dim3(256), 0, s, raw, ldr, conv, m.ring, g.ldc,            \
                        static_cast<T*>(q), static_cast<T*>(m.k), static_cast<T*>(m.vt), g.heads, g.kv_heads, g.dim, \
-                       g.vdim, g.D, g.cap, channels, M, pos0);                                                     \
+                       g.vdim, g.D, g.cap, channels, M, pos0, 0, 0, nullptr, nullptr);                             \
     break
   switch (g.taps > 0 ? g.taps : 1) {
     W4_QKV(1); W4_QKV(2); W4_QKV(3); W4_QKV(4); W4_QKV(5); W4_QKV(6); W4_QKV(7); W4_QKV(8);
@@ -704,17 +761,17 @@ hipError_t qkv_t(const AttnGeom& g, const AttnMem& m, const float* raw, int ldr,
   return hipGetLastError();
 }
 
-template <int D>
-hipError_t mfma_d(const AttnGeom& g, const AttnMem& m, const void* q, void* out, int ldo, int M, int pos0,
-                  hipStream_t s) {
-  auto kern = attn_mfma_kernel<D>;
-  constexpr size_t lds = (D / 16) * 64 * 16 + sizeof(float) * (kMfmaWaves - 1) * (D / 2 + 2) * 64;
+template <int D, int KR>
+hipError_t mfma_d(const AttnGeom& g, const AttnMem& m, const PrefillExtra& x, const void* q, void* out, int ldo, int M,
+                  int pos0, hipStream_t s) {
+  auto kern = attn_mfma_kernel<D, KR>;
+  constexpr size_t lds = (D / 16 + KR) * 64 * 16 + sizeof(float) * (kMfmaWaves - 1) * (D / 2 + 2) * 64;
   static LdsLimitOnce raised;
   if (hipError_t e = raised.raise(reinterpret_cast<const void*>(kern), lds); e != hipSuccess) return e;
   hipLaunchKernelGGL(kern, dim3(g.heads, (M + 31) / 32), dim3(64 * kMfmaWaves), lds, s, static_cast<const __bf16*>(q),
                      static_cast<const __bf16*>(m.k), static_cast<const __bf16*>(m.vt),
                      static_cast<const __bf16*>(m.kp), static_cast<const __bf16*>(m.vpt), static_cast<__bf16*>(out), ldo,
-                     M, g.heads, g.kv_heads, g.dim, g.vdim, g.cap, g.capp, g.window, g.pool, pos0, g.scale);
+                     M, g.heads, g.kv_heads, g.dim, g.vdim, g.cap, g.capp, g.window, g.pool, pos0, g.scale, x);
   return hipGetLastError();
 }
 
@@ -731,7 +788,8 @@ hipError_t decode_d(const AttnGeom& g, const AttnMem& m, const float* raw, const
   hipLaunchKernelGGL(kern, dim3(attn_slices(g, max_seq), g.kv_heads), dim3(kDecThreads), lds, s, raw, conv,
                      m.ring, g.ldc, static_cast<T*>(m.k), static_cast<T*>(m.vt), static_cast<T*>(m.kp),
                      static_cast<T*>(m.vpt), o, ml, pos, max_seq, g.heads, g.kv_heads, g.dim, g.vdim, g.cap, g.capp,
-                     g.window, g.pool, g.scale, g.taps, (int)g.own_kv, (int)g.make_pool);
+                     g.window, g.pool, g.scale, g.taps, (int)g.own_kv, (int)g.make_pool, (int)g.tied, g.rot_dims, g.sin_t, g.cos_t,
+                     g.sinks);
   return hipGetLastError();
 }
 
@@ -752,7 +810,7 @@ hipError_t decode_t(const AttnGeom& g, const AttnMem& m, const float* raw, const
 int attn_slices(const AttnGeom& g, int max_seq) {
   // four blocks of 32 entries a slice, what one pass of the kernel's value threads takes at D = 128; more slices would
   // cost the merge more than they save
-  const int blocks = std::min(g.window, max_seq) / 32 + 2 + max_seq / g.pool / 32 + 1;
+  const int blocks = std::min(g.window, max_seq) / 32 + 2 + (g.pool > 0 ? max_seq / g.pool / 32 + 1 : 0);
   return std::min(std::max((blocks + 3) / 4, 4), kPoolAttnSlices);
 }
 
@@ -780,22 +838,71 @@ hipError_t launch_attn_pool(int dtype, const AttnGeom& g, const AttnMem& m, int 
   return hipGetLastError();
 }
 
-hipError_t launch_attn_prefill(int dtype, const AttnGeom& g, const AttnMem& m, const void* q, void* out, int ldo, int M,
-                               int pos0, hipStream_t s) {
-  if (dtype == W4A32_LAYERED_BF16) {
-    switch (g.D) {
-      case 32: return mfma_d<32>(g, m, q, out, ldo, M, pos0, s);
-      case 64: return mfma_d<64>(g, m, q, out, ldo, M, pos0, s);
-      case 128: return mfma_d<128>(g, m, q, out, ldo, M, pos0, s);
-      case 256: return mfma_d<256>(g, m, q, out, ldo, M, pos0, s);
-      default: return hipErrorInvalidValue;
-    }
+template <int KR>
+static hipError_t prefill_bf16(const AttnGeom& g, const AttnMem& m, const PrefillExtra& x, const void* q, void* out, int ldo,
+                               int M, int pos0, hipStream_t s) {
+  switch (g.D) {
+    case 32: return mfma_d<32, KR>(g, m, x, q, out, ldo, M, pos0, s);
+    case 64: return mfma_d<64, KR>(g, m, x, q, out, ldo, M, pos0, s);
+    case 128: return mfma_d<128, KR>(g, m, x, q, out, ldo, M, pos0, s);
+    case 256: return mfma_d<256, KR>(g, m, x, q, out, ldo, M, pos0, s);
+    default: return hipErrorInvalidValue;
   }
+}
+
+static hipError_t prefill_f32(const AttnGeom& g, const AttnMem& m, const PrefillExtra& x, const void* q, void* out, int ldo,
+                              int M, int pos0, hipStream_t s) {
   hipLaunchKernelGGL(attn_rows_kernel<float>, dim3(g.heads, M), dim3(64), 0, s, static_cast<const float*>(q),
                      static_cast<const float*>(m.k), static_cast<const float*>(m.vt), static_cast<const float*>(m.kp),
                      static_cast<const float*>(m.vpt), static_cast<float*>(out), ldo, g.heads, g.kv_heads, g.dim, g.vdim,
-                     g.D, g.cap, g.capp, g.window, g.pool, pos0, g.scale);
+                     g.D, g.cap, g.capp, g.window, g.pool, pos0, g.scale, x);
   return hipGetLastError();
+}
+
+hipError_t launch_attn_prefill(int dtype, const AttnGeom& g, const AttnMem& m, const void* q, void* out, int ldo, int M,
+                               int pos0, hipStream_t s) {
+  PrefillExtra x{};
+  x.sinks = g.sinks;
+  x.qld = g.heads * g.D;
+  x.qstride = g.D;
+  if (dtype == W4A32_LAYERED_BF16) return prefill_bf16<0>(g, m, x, q, out, ldo, M, pos0, s);
+  return prefill_f32(g, m, x, q, out, ldo, M, pos0, s);
+}
+
+int latent_rot_pad(int rot_part) { return rot_part <= 16 ? 16 : rot_part <= 32 ? 32 : rot_part <= 64 ? 64 : 128; }
+
+hipError_t launch_latent_prefill(int dtype, const LatentGeom& g, const void* k, const void* ke, const void* ve, int nblk,
+                                 const void* q, int ldq, const float* raw, void* out, int ldo, int M, int pos0,
+                                 hipStream_t s) {
+  const size_t elem = dtype == W4A32_LAYERED_BF16 ? 2 : 4;
+  AttnGeom a{};  // every head has expanded keys and values of its own
+  a.heads = a.kv_heads = g.heads;
+  a.dim = g.dim; a.vdim = g.vdim; a.D = g.D;
+  a.cap = 32 * nblk; a.capp = 32;
+  a.window = g.window;
+  a.scale = g.scale;
+  const AttnMem m{const_cast<void*>(ke), const_cast<void*>(ve), nullptr, nullptr, nullptr};
+  PrefillExtra x{};
+  x.sinks = g.sinks;
+  x.gate = g.gate_off >= 0 ? raw + g.gate_off : nullptr;
+  x.ldg = g.ldr;
+  x.qld = ldq;
+  x.qstride = g.dim + g.rot_part;
+  x.blk0 = std::max(0, pos0 - g.window + 1) / 32;
+  x.kr = static_cast<const uint8_t*>(k) + elem * 32 * g.Dc;  // behind a block's latents
+  x.kr_block = (size_t)32 * (g.Dc + g.Dr);
+  x.rot_part = g.rot_part;
+  x.rot_dims = g.rot_dims;
+  x.sin_t = g.sin_t;
+  x.cos_t = g.cos_t;
+  if (dtype != W4A32_LAYERED_BF16) return prefill_f32(a, m, x, q, out, ldo, M, pos0, s);
+  switch (g.Dr) {
+    case 16: return prefill_bf16<1>(a, m, x, q, out, ldo, M, pos0, s);
+    case 32: return prefill_bf16<2>(a, m, x, q, out, ldo, M, pos0, s);
+    case 64: return prefill_bf16<4>(a, m, x, q, out, ldo, M, pos0, s);
+    case 128: return prefill_bf16<8>(a, m, x, q, out, ldo, M, pos0, s);
+    default: return hipErrorInvalidValue;
+  }
 }
 
 hipError_t launch_attn_decode(int dtype, const AttnGeom& g, const AttnMem& m, const float* raw, const float* conv,

@@ -60,6 +60,7 @@ int main(int argc, char** argv) {
   ctx.registerBackend(hip::createHipBackend());
   auto& registry = models::CausalLMRegistry::instance();
   models::registerSuripel(registry);
+  models::registerLesarax(registry);
   models::registerQwen2(registry);
   {
     auto model = registry.load(model_dir, options);

@@ -46,7 +46,9 @@ int main(int argc, char** argv) {
   ctx.registerBackend(hip::createHostBackend());
   ctx.registerBackend(hip::createHipRuntimeBackend());
   auto& registry = models::CausalLMRegistry::instance();
-  models::registerSuripel(registry);  // the families that give logits at any place
+  // the families that give logits at any place
+  models::registerSuripel(registry);
+  models::registerLesarax(registry);
   {
     auto model = registry.load(model_dir, options);
     std::map<std::string, int32_t> live;

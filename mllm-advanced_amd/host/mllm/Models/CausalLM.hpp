@@ -59,6 +59,7 @@ class CausalLMRegistry {
 
 // Model families register themselves by calling these (explicitly: a program links the families it names).
 void registerSuripel(CausalLMRegistry& r);
+void registerLesarax(CausalLMRegistry& r);
 void registerQwen2(CausalLMRegistry& r);
 
 }  // namespace mllm::models

@@ -85,26 +85,78 @@ const void* LayeredWeights::upload(const std::vector<uint8_t>& bytes) {
   return d.ptr<void>();
 }
 
+void LayeredWeights::copy(uint8_t* dst, const Tensor& t, size_t src, int32_t n) const {
+  if (dtype_ == W4A32_LAYERED_BF16) {
+    auto* d = reinterpret_cast<uint16_t*>(dst);
+    if (t.dtype() == kBF16) {
+      std::memcpy(d, t.ptr<uint16_t>() + src, static_cast<size_t>(n) * 2);
+    } else {
+      for (int32_t c = 0; c < n; ++c) d[c] = floatToBf16(elementAsFloat(t, src + c));
+    }
+  } else {
+    for (int32_t c = 0; c < n; ++c) reinterpret_cast<float*>(dst)[c] = elementAsFloat(t, src + c);
+  }
+}
+
 const void* LayeredWeights::matrix(const std::vector<Part>& parts, int32_t in, bool pad_rows) {
   int32_t rows = 0;
   for (const auto& p : parts) rows += p.rows;
-  const size_t ld = pad64(in), elem = dtype_ == W4A32_LAYERED_BF16 ? 2 : 4;
-  std::vector<uint8_t> buf((pad_rows ? pad64(rows) : rows) * ld * elem, 0);
+  const size_t row = pad64(in) * elem();
+  std::vector<uint8_t> buf((pad_rows ? pad64(rows) : rows) * row, 0);
   size_t at = 0;
   for (const auto& p : parts) {
     Tensor t = host(p.name, {p.rows, in});
-    for (int32_t r = 0; r < p.rows; ++r, ++at) {
-      uint8_t* dst = buf.data() + at * ld * elem;
-      const size_t src = static_cast<size_t>(r) * in;
-      if (t.dtype() == kBF16 && elem == 2) {
-        std::memcpy(dst, t.ptr<uint16_t>() + src, static_cast<size_t>(in) * 2);
-      } else if (elem == 2) {
-        for (int32_t c = 0; c < in; ++c) reinterpret_cast<uint16_t*>(dst)[c] = floatToBf16(elementAsFloat(t, src + c));
-      } else {
-        for (int32_t c = 0; c < in; ++c) reinterpret_cast<float*>(dst)[c] = elementAsFloat(t, src + c);
+    for (int32_t r = 0; r < p.rows; ++r, ++at) copy(buf.data() + at * row, t, static_cast<size_t>(r) * in, in);
+  }
+  return upload(buf);
+}
+
+const void* LayeredWeights::operandBlocks(const std::string& name, int32_t heads, int32_t n, int32_t head_rows, int32_t in) {
+  const size_t ld = pad64(in);
+  std::vector<uint8_t> buf(static_cast<size_t>(heads) * head_rows * ld * elem(), 0);
+  Tensor t = host(name, {heads * n, in});
+  for (int32_t h = 0; h < heads; ++h)
+    for (int32_t i = 0; i < n; ++i) {
+      const size_t r = static_cast<size_t>(h) * head_rows + i;
+      for (int32_t c = 0; c < in; c += 8) {
+        const size_t at = ((r / 32 * (ld / 8) + c / 8) * 32 + r % 32) * 8;
+        copy(buf.data() + at * elem(), t, (static_cast<size_t>(h) * n + i) * in + c, std::min(8, in - c));
       }
     }
+  return upload(buf);
+}
+
+const void* LayeredWeights::gateUp(const std::vector<std::pair<std::string, std::string>>& experts, int32_t ff, int32_t in) {
+  const size_t row = pad64(in) * elem(), rows = 2 * pad64(ff);
+  std::vector<uint8_t> buf(experts.size() * rows * row, 0);
+  for (size_t e = 0; e < experts.size(); ++e) {
+    Tensor gate = host(experts[e].first, {ff, in}), up = host(experts[e].second, {ff, in});
+    for (int32_t r = 0; r < ff; ++r) {
+      uint8_t* dst = buf.data() + (e * rows + r / 32 * 64 + r % 32) * row;
+      copy(dst, gate, static_cast<size_t>(r) * in, in);
+      copy(dst + 32 * row, up, static_cast<size_t>(r) * in, in);
+    }
   }
+  return upload(buf);
+}
+
+const void* LayeredWeights::stack(const std::vector<std::string>& names, int32_t out, int32_t in) {
+  const size_t row = pad64(in) * elem(), rows = pad64(out);
+  std::vector<uint8_t> buf(names.size() * rows * row, 0);
+  for (size_t e = 0; e < names.size(); ++e) {
+    Tensor t = host(names[e], {out, in});
+    for (int32_t r = 0; r < out; ++r) copy(buf.data() + (e * rows + r) * row, t, static_cast<size_t>(r) * in, in);
+  }
+  return upload(buf);
+}
+
+const void* LayeredWeights::halves(const std::string& name, int32_t out, int32_t in) {
+  const size_t half = pad64(in) * elem();
+  std::vector<uint8_t> buf(pad64(out) * 2 * half, 0);
+  Tensor t = host(name, {out, 2 * in});
+  for (int32_t r = 0; r < out; ++r)
+    for (int32_t i = 0; i < 2; ++i)
+      copy(buf.data() + (2 * static_cast<size_t>(r) + i) * half, t, (2 * static_cast<size_t>(r) + i) * in, in);
   return upload(buf);
 }
 
@@ -159,6 +211,11 @@ HipLayeredForCausalLM::HipLayeredForCausalLM(const LayeredSpec& spec, const Caus
   cfg_.canon_taps = spec.canon_taps;
   cfg_.norm_eps = spec.norm_eps;
   cfg_.dtype = spec.dtype;
+  cfg_.norm = spec.norm;
+  cfg_.residual_mult = spec.residual_mult;
+  cfg_.loop_start = spec.loop_start;
+  cfg_.loop_stop = spec.loop_stop;
+  cfg_.loop_times = spec.loop_times;
   cfg_.max_seq = std::max(options.max_tokens, 1);
   cfg_.max_batch_tokens = std::max(1, std::min(options.max_chunk, cfg_.max_seq));
   cfg_.layers = layer_cfg_.data();

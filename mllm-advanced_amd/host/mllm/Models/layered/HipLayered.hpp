@@ -1,13 +1,14 @@
 // A decoder-only model whose layers are described one by one, on the layered decoder runner
 // (include/w4a32_layered.h). The class owns the device memory (weights, workspace, one state per sequence) and the
-// captured decode step; a design's own file (mllm/Models/suripel) reads its configuration and parameter names and fills in the
-// specification and the weights through LayeredWeights.
+// captured decode step; a design's own file (mllm/Models/suripel, mllm/Models/lesarax) reads its configuration and
+// parameter names and fills in the specification and the weights through LayeredWeights.
 #pragma once
 
 #include <cstdint>
 #include <map>
 #include <memory>
 #include <string>
+#include <utility>
 #include <vector>
 
 #include "mllm/Core/Tensor.hpp"
@@ -22,6 +23,9 @@ struct LayeredSpec {
   float norm_eps = 1e-5f;
   int dtype = W4A32_LAYERED_BF16;
   std::vector<w4a32_layer_config> layers;
+  int norm = W4A32_NORM_LAYER;
+  float residual_mult = 1.0f;
+  int32_t loop_start = 0, loop_stop = 0, loop_times = 0;
 };
 
 // Host parameters (BF16, Fp16 or Fp32) -> device memory in the runner's layouts. Every tensor's shape is checked
@@ -36,6 +40,14 @@ class LayeredWeights {
   };
   // [out, in] matrices one below the other, in the model's element type. pad_rows: rows to a multiple of 64 as well.
   const void* matrix(const std::vector<Part>& parts, int32_t in, bool pad_rows = true);
+  // [heads * n, in] as operand blocks (w4a32_layered.h): head_rows rows per head, the true ones first
+  const void* operandBlocks(const std::string& name, int32_t heads, int32_t n, int32_t head_rows, int32_t in);
+  // experts' gate and up [ff, in], one pair of names per expert, in groups of 32 rows of each
+  const void* gateUp(const std::vector<std::pair<std::string, std::string>>& experts, int32_t ff, int32_t in);
+  // equal matrices [out, in] one behind the other, each padded by itself
+  const void* stack(const std::vector<std::string>& names, int32_t out, int32_t in);
+  // [out, 2 in] whose two column halves are padded each
+  const void* halves(const std::string& name, int32_t out, int32_t in);
   // a vector, f32
   const float* vector(const std::string& name, int32_t n);
   const float* values(const std::vector<float>& v);
@@ -45,6 +57,9 @@ class LayeredWeights {
  private:
   Tensor host(const std::string& name, const std::vector<int32_t>& shape);
   const void* upload(const std::vector<uint8_t>& bytes);
+  [[nodiscard]] size_t elem() const { return dtype_ == W4A32_LAYERED_BF16 ? 2 : 4; }
+  // n elements from element `src` of t on, in the model's element type
+  void copy(uint8_t* dst, const Tensor& t, size_t src, int32_t n) const;
 
   std::shared_ptr<ParameterLoader> file_;
   int dtype_;
