@@ -78,6 +78,70 @@ def random_weights(cfg, seed=0):
     return w
 
 
+# ---------------------------------------------------------------------------------------------- Lesarax
+def moe(ff, experts, top, limit=1.2):
+    return {"kind": "moe", "expert": {"ff": ff, "limit": float(limit)}, "router": {"experts": experts, "top": top}}
+
+
+def rotary(heads, kv_heads, dim, rot, base=7000.0, scale=None, mlp=None):
+    return {"type": "attention", "mlp": mlp,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
+                      "scale": float(scale if scale is not None else dim ** -0.5), "rot": {"dims": rot, "base": base}}}
+
+
+def latent(heads, dim, rot_dim, vdim, q_rank, kv_rank, size, base=3000.0, scale=None, mlp=None):
+    return {"type": "latent_attention", "mlp": mlp,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+                      "scale": float(scale if scale is not None else (dim + rot_dim) ** -0.5), "mask": {"size": size},
+                      "rot": {"dims": rot_dim, "base": base}}}
+
+
+def lesarax(layers, width=104, vocab=59, loop=(0, 1, 1), mult=0.7, eps=EPS):
+    return {"architecture": "Lesarax", "width": width, "vocab": vocab, "norm": {"eps": eps}, "residual_mult": mult,
+            "loop": dict(zip(("start", "stop", "times"), loop)), "layers": layers}
+
+
+def lesarax_weights(cfg, seed=0):
+    rng = np.random.default_rng(seed)
+    W = cfg["width"]
+    w = {}
+
+    def put(name, *shape, std=None, mean=0.0):
+        std = shape[-1] ** -0.5 if std is None else std
+        w[name] = lo.bf16_round(rng.standard_normal(shape) * std + mean)
+
+    put("embed", cfg["vocab"], W, std=1.0)
+    put("final.norm", W, std=0.2, mean=1.0)
+    put("loop.in", W, 2 * W)
+    for i, layer in enumerate(cfg["layers"]):
+        p, q, m = f"l{i}.", f"l{i}.mix.", layer["mixer"]
+        H = m["heads"]
+        put(p + "norm1", W, std=0.2, mean=1.0)
+        if layer["type"] == "attention":
+            put(q + "q", H * m["dim"], W, std=1.5 * W ** -0.5)
+            put(q + "k", m["kv_heads"] * m["dim"], W, std=1.5 * W ** -0.5)
+        else:
+            put(q + "dq", m["q_rank"], W)
+            put(q + "dq.norm", m["q_rank"], std=0.2, mean=1.0)
+            put(q + "uq", H * (m["dim"] + m["rot_dim"]), m["q_rank"], std=1.5 * m["q_rank"] ** -0.5)
+            put(q + "dkv", m["kv_rank"] + m["rot_dim"], W)
+            put(q + "dkv.norm", m["kv_rank"], std=0.2, mean=1.0)
+            put(q + "uk", H * m["dim"], m["kv_rank"])
+            put(q + "uv", H * m["vdim"], m["kv_rank"])
+            put(q + "g", H, W, std=2 * W ** -0.5)
+        put(q + "sink", H, std=1.0, mean=1.0)
+        put(q + "o", W, H * m["vdim"])
+        if layer["mlp"]:
+            E, F = layer["mlp"]["router"]["experts"], layer["mlp"]["expert"]["ff"]
+            put(p + "norm2", W, std=0.2, mean=1.0)
+            put(p + "mlp.router", E, W, std=2 * W ** -0.5)
+            for e in range(E):
+                put(f"{p}mlp.e{e}.gate", F, W, std=1.5 * W ** -0.5)
+                put(f"{p}mlp.e{e}.up", F, W, std=1.5 * W ** -0.5)
+                put(f"{p}mlp.e{e}.down", W, F)
+    return w
+
+
 def runner(cfg, w, dtype, max_seq, max_batch_tokens=None):
     import torch
 
