@@ -72,8 +72,11 @@ def parse():
                     help="instead of the default workload: prefill and decode of the layered decoder (pooled-window "
                          "attention / gated delta rule / retention, bf16) beside the W4A32 decoder of equal size; "
                          "SIZES: comma-separated names of LAYERED_SIZES")
-    ap.add_argument("--layered-only", choices=("both", "layered", "w4a32"), default="both",
-                    help="with --layered: run one of the two models (for a profile of it alone)")
+    ap.add_argument("--lesarax", metavar="SIZES", nargs="?", const="small,mid,large", default=None,
+                    help="instead of the default workload: prefill and decode of a decoder with latent and rotary attention, "
+                         "experts and looped layers (bf16) beside the layered decoder of equal size; SIZES as for --layered")
+    ap.add_argument("--layered-only", choices=("both", "layered", "w4a32", "lesarax"), default="both",
+                    help="with --layered or --lesarax: run one of the two models (for a profile of it alone)")
     return ap.parse_args()
 
 
@@ -138,6 +141,52 @@ def layered_model(torch, size, gen):
     return cfg, w, matrix
 
 
+def lesarax_model(torch, size, gen):
+    """As layered_model for Lesarax: as many layer runs (the middle half of them two passes through a quarter of the layers),
+    three latent layers to one of rotary attention, 16 experts of a quarter of the feed-forward's width of which 4 run."""
+    W, H, G, F, L, V = size
+    q_rank, kv_rank, rot = W // 2, 512 if W > 2000 else 256, 64
+    start = quarter = L // 4
+    n = L - quarter
+    mlp = {"kind": "moe", "expert": {"ff": F // 4, "limit": 7.0}, "router": {"experts": 16, "top": 4}}
+    layers = []
+    for i in range(n):
+        if i % 4 == 2:
+            m = {"heads": H, "kv_heads": G, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "rot": {"dims": rot, "base": 1e6}}
+            layers.append({"type": "attention", "mixer": m, "mlp": mlp})
+        else:
+            m = {"heads": H, "dim": 128, "rot_dim": rot, "vdim": 128, "q_rank": q_rank, "kv_rank": kv_rank,
+                 "scale": (128 + rot) ** -0.5, "mask": {"size": 1024}, "rot": {"dims": rot, "base": 1e6}}
+            layers.append({"type": "latent_attention", "mixer": m, "mlp": mlp})
+    cfg = {"architecture": "Lesarax", "width": W, "vocab": V, "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+           "loop": {"start": start, "stop": start + quarter, "times": 2}, "layers": layers}
+
+    def rnd(*shape, std=0.02):
+        return (torch.randn(shape, generator=gen, device="cuda") * std).to(torch.bfloat16)
+    one = lambda n: torch.ones(n, device="cuda")
+    w = {"embed": rnd(V, W, std=1.0), "final.norm": one(W), "loop.in": rnd(W, 2 * W)}
+    body = 0                                    # elements of the matrices one token meets in the layers' runs
+    for i, layer in enumerate(layers):
+        m, p, q = layer["mixer"], f"l{i}.", f"l{i}.mix."
+        if layer["type"] == "attention":
+            shapes = {"q": (H * 128, W), "k": (G * 128, W)}
+        else:
+            shapes = {"dq": (q_rank, W), "uq": (H * (128 + rot), q_rank), "dkv": (kv_rank + rot, W),
+                      "uk": (H * 128, kv_rank), "uv": (H * 128, kv_rank), "g": (H, W)}
+            w[q + "dq.norm"], w[q + "dkv.norm"] = one(q_rank), one(kv_rank)
+        shapes["o"] = (W, H * 128)
+        for name, shape in shapes.items():
+            w[q + name] = rnd(*shape)
+        w[q + "sink"] = rnd(H, std=1.0)
+        w[p + "norm1"], w[p + "norm2"], w[p + "mlp.router"] = one(W), one(W), rnd(16, W)
+        for e in range(16):
+            w[f"{p}mlp.e{e}.gate"], w[f"{p}mlp.e{e}.up"] = rnd(F // 4, W), rnd(F // 4, W)
+            w[f"{p}mlp.e{e}.down"] = rnd(W, F // 4)
+        runs = 2 if start <= i < start + quarter else 1
+        body += runs * (sum(a * b for a, b in shapes.values()) + 16 * W + 3 * F * W)
+    return cfg, w, body + 2 * 2 * W * W + V * W
+
+
 def layered_bench(args, torch, pkg):
     gen = torch.Generator(device="cuda")
     gen.manual_seed(7)
@@ -148,6 +197,7 @@ def layered_bench(args, torch, pkg):
     def measure(prefill, step, prepare):
         """ms per prefill of each length, ms per greedy step behind a 2048-token prompt (graph replay)."""
         out = {}
+        torch.cuda.synchronize()                # weights and workspace are made on the default stream
         with torch.cuda.stream(stream):
             for n in prompts:
                 ids = torch.randint(0, 1000, (n,), generator=gen, device="cuda", dtype=torch.int64)
@@ -177,18 +227,22 @@ def layered_bench(args, torch, pkg):
         return out
 
     rows = {}
-    for name in args.layered.split(","):
+    makers = {"layered": layered_model, "lesarax": lesarax_model}
+    models = ("lesarax", "layered") if args.lesarax else ("layered", "w4a32")
+    if args.layered_only != "both":
+        models = tuple(m for m in models if m == args.layered_only)
+    for name in (args.lesarax or args.layered).split(","):
         size = LAYERED_SIZES[name]
         W, H, G, F, L, V = size
         row = {"size": dict(zip(("hidden", "heads", "kv_heads", "ff", "layers", "vocab"), size))}
-        if args.layered_only != "w4a32":
-            cfg, w, matrix = layered_model(torch, size, gen)
+        for kind in (m for m in models if m in makers):
+            cfg, w, matrix = makers[kind](torch, size, gen)
             dec = pkg.LayeredDecoder(cfg, w, "bfloat16", max_seq=max_seq, max_batch_tokens=max(prompts))
             del w
             st = dec.new_state()
             t = measure(lambda ids: dec.prefill(st, ids), lambda: dec.step(st), lambda ids: dec.prefill(st, ids))
             body = matrix - V * W
-            row["layered"] = {
+            row[kind] = {
                 **{f"prefill_ms_{n}": round(t[n], 3) for n in prompts},
                 **{f"prefill_tokens_per_s_{n}": round(n / t[n] * 1e3) for n in prompts},
                 # matrix products alone, against the dense bf16 peak
@@ -196,7 +250,7 @@ def layered_bench(args, torch, pkg):
                 "decode_ms": round(t["decode"], 4), "decode_tokens_per_s": round(1e3 / t["decode"], 1),
                 "decode_weight_bytes": 2 * matrix, "decode_GBps": round(2e-6 * matrix / t["decode"], 1)}
             del dec, st
-        if args.layered_only != "layered":
+        if "w4a32" in models:
             shapes = {"q": (W, H * 128), "k": (W, G * 128), "v": (W, G * 128), "o": (H * 128, W), "gate": (W, F),
                       "up": (W, F), "down": (F, W)}
             pack = lambda K, N: pkg.quant_pack_rhs(torch.randn((N, K), generator=gen, device="cuda") * 0.02)
@@ -220,8 +274,9 @@ def layered_bench(args, torch, pkg):
         torch.cuda.empty_cache()
         rows[name] = row
         print(f"# {name}: {json.dumps(row)}", file=sys.stderr, flush=True)
-    print(json.dumps({"metric": "layered decoder beside the W4A32 decoder", "unit": "ms, tokens/s", "n_gpus": 1,
-                      "data": "synthetic", "dtype": "bf16 (layered), W4A32 (w4a32)", "prompt_for_decode": max(prompts),
+    title = "Lesarax beside the layered decoder" if args.lesarax else "layered decoder beside the W4A32 decoder"
+    print(json.dumps({"metric": title, "unit": "ms, tokens/s", "n_gpus": 1,
+                      "data": "synthetic", "dtype": "bf16" if args.lesarax else "bf16 (layered), W4A32 (w4a32)", "prompt_for_decode": max(prompts),
                       "decode_steps": n_new, "sizes": rows}))
 
 
@@ -249,7 +304,7 @@ def main():
     L = pkg.lib()                       # raises if the HIP library is missing: no fallback
     assert torch.cuda.is_available(), "bench.py needs the MI355X"
     torch.cuda.set_device(0)
-    if args.layered:
+    if args.layered or args.lesarax:
         return layered_bench(args, torch, pkg)
     gen = torch.Generator(device="cuda")
     gen.manual_seed(0)

@@ -925,6 +925,7 @@ class LayeredDecoder:
         _check(lib().w4a32_layered_init_workspace(ctypes.byref(self.cfg), _ptr(self.ws), _stream()),
                "w4a32_layered_init_workspace")
         self.token = torch.zeros((1,), dtype=torch.int64, device="cuda")
+        torch.cuda.current_stream().synchronize()   # ready for a caller on any stream
 
     def _suripel(self, config, weights):
         import math
@@ -1040,8 +1041,11 @@ class LayeredDecoder:
 
     def new_state(self):
         """Memory of one sequence. A used one serves another sequence as it is (which starts at position 0)."""
+        import torch
+
         st = _dev_empty(int(lib().w4a32_layered_state_bytes(ctypes.byref(self.cfg))))
         _check(lib().w4a32_layered_init_state(ctypes.byref(self.cfg), _ptr(st), _stream()), "w4a32_layered_init_state")
+        torch.cuda.current_stream().synchronize()
         return st
 
     def forward(self, state, tokens, pos0, want=None):

@@ -166,6 +166,7 @@ __device__ __forceinline__ bool moe_tile(const MoeTile* __restrict__ tiles, cons
   if ((int)blockIdx.x >= total) return false;
   const int t = xcd_tile(blockIdx.x, total);
   const MoeTile any = tiles[t / nt];  // a tile of the expert
+  if (any.tiles <= 0) return false;
   const int local = t - any.first * nt;
   *tile = tiles[any.first + local % any.tiles];
   *n = local / any.tiles;
