@@ -34,18 +34,37 @@ __device__ __forceinline__ void latent_of_row(const float* __restrict__ raw, int
                                               const float* __restrict__ sin_t, const float* __restrict__ cos_t,
                                               float* __restrict__ s_c) {
   const int lane = threadIdx.x & 63;
-  float ss = 0.0f;
-  for (int d = lane; d < kv_rank; d += 64) {
-    const float x = raw[kv_off + d];
-    ss += x * x;
+  constexpr int kRegs = kMaxLatent / 64, kRotRegs = kMaxRot / 64;
+  float x[kRegs], w[kRegs], y[kRotRegs], z[kRotRegs], sn[kRotRegs], cs[kRotRegs], ss = 0.0f;
+  const int half = rot_dims / 2;
+#pragma unroll
+  for (int i = 0; i < kRotRegs; ++i) {  // all requested before the first is used
+    const int d = min(lane + 64 * i, max(rot_part - 1, 0)), angle = d < half ? d : d - half;
+    const bool turn = d < rot_dims;
+    y[i] = rot_part > 0 ? raw[rot_off + d] : 0.0f;
+    z[i] = turn ? raw[rot_off + rot_partner(d, rot_dims)] : 0.0f;
+    cs[i] = turn ? cos_t[(size_t)p * half + angle] : 1.0f;
+    sn[i] = turn ? sin_t[(size_t)p * half + angle] : 0.0f;
+    if (d < half) sn[i] = -sn[i];
+  }
+#pragma unroll
+  for (int i = 0; i < kRegs; ++i) {
+    const int d = min(lane + 64 * i, kv_rank - 1);
+    x[i] = 64 * i < kv_rank ? raw[kv_off + d] : 0.0f;
+    w[i] = 64 * i < kv_rank ? norm_w[d] : 0.0f;
+  }
+#pragma unroll
+  for (int i = 0; i < kRegs; ++i) {
+    if (lane + 64 * i >= kv_rank) x[i] = 0.0f;
+    ss += x[i] * x[i];
   }
   const float r = 1.0f / sqrtf(wave_sum64(ss) / (float)kv_rank + eps);
-  for (int d = lane; d < kv_rank; d += 64) s_c[d] = raw[kv_off + d] * r * norm_w[d];
-  for (int d = lane; d < rot_part; d += 64) {
-    float y = raw[rot_off + d];
-    if (d < rot_dims) y = rotated(y, raw[rot_off + rot_partner(d, rot_dims)], d, rot_dims, (size_t)p, sin_t, cos_t);
-    s_c[kv_rank + d] = y;
-  }
+#pragma unroll
+  for (int i = 0; i < kRegs; ++i)
+    if (lane + 64 * i < kv_rank) s_c[lane + 64 * i] = x[i] * r * w[i];
+#pragma unroll
+  for (int i = 0; i < kRotRegs; ++i)
+    if (lane + 64 * i < rot_part) s_c[kv_rank + lane + 64 * i] = y[i] * cs[i] + z[i] * sn[i];
 }
 
 struct RowsArgs {
@@ -54,30 +73,52 @@ struct RowsArgs {
   const float *q_norm, *kv_norm, *sin_t, *cos_t;
 };
 
-// A workgroup takes up to eight tokens, aligned to eight positions (a run of values of one dimension is one store).
+// A workgroup takes up to eight tokens, aligned to eight positions (a run of values of one dimension is one store), a
+// wavefront each.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restrict__ raw, T* __restrict__ cq,
-                                                          T* __restrict__ kc, T* __restrict__ vt, int M, int pos0,
-                                                          const RowsArgs a) {
+__global__ __launch_bounds__(64 * kRowTok) void latent_rows_kernel(const float* __restrict__ raw, T* __restrict__ cq,
+                                                                   T* __restrict__ kc, T* __restrict__ vt, int M, int pos0,
+                                                                   const RowsArgs a) {
   extern __shared__ __align__(16) float s_c[];  // [kRowTok][kv_rank + rot_part]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, ld = a.kv_rank + a.rot_part;
   const int lead = pos0 & (kRowTok - 1);
   const int t0 = max(0, (int)blockIdx.x * kRowTok - lead), te = min(M, ((int)blockIdx.x + 1) * kRowTok - lead);
-  for (int t = t0 + wave; t < te; t += 4) {
+  const int t = t0 + wave;
+  if (t < te) {
     const float* row = raw + (size_t)t * a.ldr;
-    float ss = 0.0f;
-    for (int d = lane; d < a.q_rank; d += 64) ss += row[d] * row[d];
-    const float r = 1.0f / sqrtf(wave_sum64(ss) / (float)a.q_rank + a.eps);
-    for (int d = lane; d < a.ldq; d += 64) cq[(size_t)t * a.ldq + d] = d < a.q_rank ? (T)(row[d] * r * a.q_norm[d]) : (T)0.0f;
-    latent_of_row(row, a.kv_rank, a.rot_part, a.rot_dims, a.kv_off, a.rot_off, a.kv_norm, a.eps, pos0 + t, a.sin_t, a.cos_t,
-                  s_c + (size_t)(t - t0) * ld);
+    constexpr int kRegs = 16;  // a query latent of up to 1024 stays in registers
+    float x[kRegs], ss = 0.0f;
+    if (a.ldq <= 64 * kRegs) {
+#pragma unroll
+      for (int i = 0; i < kRegs; ++i) x[i] = row[min(lane + 64 * i, a.q_rank - 1)];
+      latent_of_row(row, a.kv_rank, a.rot_part, a.rot_dims, a.kv_off, a.rot_off, a.kv_norm, a.eps, pos0 + t, a.sin_t,
+                    a.cos_t, s_c + (size_t)wave * ld);
+#pragma unroll
+      for (int i = 0; i < kRegs; ++i) {
+        if (lane + 64 * i >= a.q_rank) x[i] = 0.0f;
+        ss += x[i] * x[i];
+      }
+      const float r = 1.0f / sqrtf(wave_sum64(ss) / (float)a.q_rank + a.eps);
+#pragma unroll
+      for (int i = 0; i < kRegs; ++i) {
+        const int d = lane + 64 * i;
+        if (d < a.ldq) cq[(size_t)t * a.ldq + d] = (T)(x[i] * r * a.q_norm[d]);
+      }
+    } else {
+      latent_of_row(row, a.kv_rank, a.rot_part, a.rot_dims, a.kv_off, a.rot_off, a.kv_norm, a.eps, pos0 + t, a.sin_t,
+                    a.cos_t, s_c + (size_t)wave * ld);
+      for (int d = lane; d < a.q_rank; d += 64) ss += row[d] * row[d];
+      const float r = 1.0f / sqrtf(wave_sum64(ss) / (float)a.q_rank + a.eps);
+      for (int d = lane; d < a.ldq; d += 64)
+        cq[(size_t)t * a.ldq + d] = d < a.q_rank ? (T)(row[d] * r * a.q_norm[d]) : (T)0.0f;
+    }
   }
   __syncthreads();
   const int n = te - t0, p0 = pos0 + t0, D = a.Dc + a.Dr;
   T* kb = kc + (size_t)(p0 >> 5) * (32 * D);  // all of them lie in one block
   T* vb = vt + (size_t)(p0 >> 5) * (32 * a.Dc);
   // keys: the tokens of eight dimensions side by side
-  for (int it = threadIdx.x; it < (D / 8) * kRowTok; it += 256) {
+  for (int it = threadIdx.x; it < (D / 8) * kRowTok; it += 64 * kRowTok) {
     const int s = it / kRowTok, i = it & (kRowTok - 1);
     if (i >= n) continue;
     const float* src = s_c + (size_t)i * ld;
@@ -90,7 +131,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restric
     *reinterpret_cast<E8*>(kb + (size_t)(s * 32 + ((p0 + i) & 31)) * 8) = v;
   }
   // values: runs of four tokens of a dimension
-  for (int it = threadIdx.x; it < a.kv_rank * 2; it += 256) {
+  for (int it = threadIdx.x; it < a.kv_rank * 2; it += 64 * kRowTok) {
     const int d = it >> 1, first = 4 * (it & 1) - (p0 & (kRowTok - 1));  // this run's first token
     const int q = (p0 & ~(kRowTok - 1)) + 4 * (it & 1);                  // its position
     T* dst = vb + (size_t)d * 32 + v_pos(q & 31);
@@ -137,8 +178,8 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(const __bf16* __rest
     for (int c = 0; c < 2; ++c)
 #pragma unroll
       for (int v = 0; v < 16; ++v) acc[i][c][v] = 0.0f;
-  // four steps of 16 latent dimensions at a time (Dc is a multiple of 64), the next four on their way
-  bf16x8 wf[2][2][4], cf[2][2][4];  // [register set][block][step]
+  // four steps of 16 latent dimensions at a time (Dc is a multiple of 64), the next eight on their way
+  bf16x8 wf[3][2][4], cf[3][2][4];  // [register set][block][step]
   auto fetch = [&](int s, int set) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < 2; ++i)
@@ -147,6 +188,7 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(const __bf16* __rest
         wf[set][i][u] = *reinterpret_cast<const bf16x8*>(wa[i] + 512 * (s + u));
         cf[set][i][u] = *reinterpret_cast<const bf16x8*>(ca[i] + 512 * (s + u));
       }
+    __builtin_amdgcn_sched_barrier(0);  // or the loads sink to their uses
   };
   auto products = [&](auto keys, int set) __attribute__((always_inline)) {
 #pragma unroll
@@ -160,12 +202,16 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(const __bf16* __rest
   };
   auto all = [&](auto keys) __attribute__((always_inline)) {
     fetch(0, 0);
-    for (int s = 0; s < KS; s += 8) {
-      fetch(min(s + 4, KS - 4), 1);
+    fetch(min(4, KS - 4), 1);
+    for (int s = 0; s < KS; s += 12) {
+      fetch(min(s + 8, KS - 4), 2);
       products(keys, 0);
       if (s + 4 >= KS) break;
-      fetch(min(s + 8, KS - 4), 0);
+      fetch(min(s + 12, KS - 4), 0);
       products(keys, 1);
+      if (s + 8 >= KS) break;
+      fetch(min(s + 16, KS - 4), 1);
+      products(keys, 2);
     }
   };
   const int per_head = D / 32;
@@ -321,9 +367,9 @@ __global__ __launch_bounds__(64 * kDecWaves) void latent_decode_kernel(
     const int* __restrict__ d_pos, int max_seq, int heads, int Dc, int Dr, int window, float scale,
     const float* __restrict__ sinks, float* __restrict__ o, float* __restrict__ ml) {
   extern __shared__ __align__(16) uint8_t smem[];
-  const int D = Dc + Dr, KS = D / 16, DB = Dc / 32, KS8 = (KS + 7) & ~7;
-  bf16x8* s_q = reinterpret_cast<bf16x8*>(smem);                   // [KS8][64], zeros past KS
-  bf16x8* s_p = s_q + (size_t)KS8 * 64;                            // [waves][ks][term][64]
+  const int D = Dc + Dr, KS = D / 16, DB = Dc / 32;
+  bf16x8* s_q = reinterpret_cast<bf16x8*>(smem);                   // [8 (CW + 1)][64], zeros past KS
+  bf16x8* s_p = s_q + 8 * (CW + 1) * 64;                            // [waves][ks][term][64]
   float* s_max = reinterpret_cast<float*>(s_p + kDecWaves * 4 * 64);  // [2][waves][32]
   float* s_sum = s_max + 2 * kDecWaves * 32;                       // [waves][32]
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, j = lane & 31, hh = lane >> 5;
@@ -332,17 +378,49 @@ __global__ __launch_bounds__(64 * kDecWaves) void latent_decode_kernel(
   int lo, b_lo, b_hi;
   slice_blocks(p, window, gridDim.x, slice, &lo, &b_lo, &b_hi);
 
+  // A tile's operands are requested as a whole: this wavefront's block of keys, its latent dimensions of all blocks.
+  constexpr int KQ = 8 * (CW + 1);  // most steps of 16 dimensions: Dc up to 128 CW, Dr up to 128
   const __bf16* kb = kc + 8 * lane;
   const __bf16* vb = vt + 32 * j + 8 * hh;
-  for (int it = threadIdx.x; it < KS8 * 64; it += 64 * kDecWaves) {
-    const int s = it >> 6, l = it & 63, h = 32 * (int)blockIdx.y + (l & 31);
-    const float* src = qa + (size_t)min(h, heads - 1) * D + 16 * min(s, KS - 1) + 8 * (l >> 5);
-    float4 x0 = load4(src), x1 = load4(src + 4);
-    if (s >= KS) x0 = x1 = make_float4(0, 0, 0, 0);
+  bf16x8 kop[KQ], vop[kDecWaves][CW][2];
+  auto load_k = [&](int bt) __attribute__((always_inline)) {
+    const __bf16* src = kb + (size_t)min(bt + wave, b_hi - 1) * 32 * D;
+#pragma unroll
+    for (int s = 0; s < KQ; ++s) kop[s] = *reinterpret_cast<const bf16x8*>(src + 512 * min(s, KS - 1));
+  };
+  auto load_v = [&](int bt) __attribute__((always_inline)) {
+#pragma unroll
+    for (int w = 0; w < kDecWaves; ++w)
+#pragma unroll
+      for (int i = 0; i < CW; ++i)
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks)
+          vop[w][i][ks] = *reinterpret_cast<const bf16x8*>(
+              vb + ((size_t)min(bt + w, b_hi - 1) * Dc + 32 * min(wave + kDecWaves * i, DB - 1)) * 32 + 16 * ks);
+  };
+  constexpr int NQ = 2 * (CW + 1);  // pieces of the query operands a thread brings
+  float4 qx[NQ][2];
+#pragma unroll
+  for (int i = 0; i < NQ; ++i) {
+    const int s = wave + kDecWaves * i, h = min(head, heads - 1);
+    const float* src = qa + (size_t)h * D + 16 * min(s, KS - 1) + 8 * hh;
+    qx[i][0] = load4(src);
+    qx[i][1] = load4(src + 4);
+  }
+  constexpr bool kAhead = CW <= 2;  // registers for both
+  if (b_lo < b_hi) {
+    load_k(b_lo);
+    if (kAhead) load_v(b_lo);
+  }
+  __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+  for (int i = 0; i < NQ; ++i) {
+    const int s = wave + kDecWaves * i;
+    const float x[8] = {qx[i][0].x, qx[i][0].y, qx[i][0].z, qx[i][0].w, qx[i][1].x, qx[i][1].y, qx[i][1].z, qx[i][1].w};
     bf16x8 v;
-    v[0] = (__bf16)x0.x; v[1] = (__bf16)x0.y; v[2] = (__bf16)x0.z; v[3] = (__bf16)x0.w;
-    v[4] = (__bf16)x1.x; v[5] = (__bf16)x1.y; v[6] = (__bf16)x1.z; v[7] = (__bf16)x1.w;
-    s_q[it] = v;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = s < KS ? (__bf16)x[e] : (__bf16)0.0f;
+    s_q[s * 64 + lane] = v;
   }
   f32x16 acc[CW];
 #pragma unroll
@@ -365,26 +443,10 @@ __global__ __launch_bounds__(64 * kDecWaves) void latent_decode_kernel(
     for (int v = 0; v < 16; ++v) st[v] = st1[v] = 0.0f;
     if (wave < n) {
       const int b = bt + wave;
-      const __bf16* src = kb + (size_t)b * 32 * D;
-      bf16x8 kop[2][8];
-      auto fetch = [&](int s, bf16x8 (&k)[8]) __attribute__((always_inline)) {
 #pragma unroll
-        for (int u = 0; u < 8; ++u) k[u] = *reinterpret_cast<const bf16x8*>(src + 512 * min(s + u, KS - 1));
-      };
-      auto products = [&](int s, const bf16x8 (&k)[8]) __attribute__((always_inline)) {
-#pragma unroll
-        for (int u = 0; u < 8; u += 2) {
-          st = mfma_bf16(k[u], s_q[(s + u) * 64 + lane], st);
-          st1 = mfma_bf16(k[u + 1], s_q[(s + u + 1) * 64 + lane], st1);
-        }
-      };
-      fetch(0, kop[0]);
-      for (int s = 0; s < KS; s += 16) {
-        fetch(s + 8, kop[1]);
-        products(s, kop[0]);
-        if (s + 8 >= KS) break;
-        fetch(s + 16, kop[0]);
-        products(s + 8, kop[1]);
+      for (int s = 0; s < KQ; s += 2) {
+        st = mfma_bf16(kop[s], s_q[s * 64 + lane], st);
+        st1 = mfma_bf16(kop[s + 1], s_q[(s + 1) * 64 + lane], st1);
       }
 #pragma unroll
       for (int v = 0; v < 16; ++v) {
@@ -394,6 +456,7 @@ __global__ __launch_bounds__(64 * kDecWaves) void latent_decode_kernel(
       }
       blk_max = fmaxf(blk_max, __shfl_xor(blk_max, 32, 64));
     }
+    if (!kAhead) load_v(bt);
     float* mx = s_max + turn * kDecWaves * 32;
     if (hh == 0) mx[wave * 32 + j] = blk_max;
     __syncthreads();
@@ -429,33 +492,31 @@ __global__ __launch_bounds__(64 * kDecWaves) void latent_decode_kernel(
     for (int i = 0; i < CW; ++i)
 #pragma unroll
       for (int v = 0; v < 16; ++v) acc[i][v] *= corr;
-    for (int w = 0; w < n; ++w) {
+#pragma unroll
+    for (int w = 0; w < kDecWaves; ++w) {
+      if (w >= n) break;
       const int b = bt + w;
-      const bool edge = 32 * b + 31 > p;
-      bf16x8 vop[CW][2];
-#pragma unroll
-      for (int i = 0; i < CW; ++i)
-#pragma unroll
-        for (int ks = 0; ks < 2; ++ks)
-          vop[i][ks] = *reinterpret_cast<const bf16x8*>(vb + ((size_t)b * Dc + 32 * min(wave + kDecWaves * i, DB - 1)) * 32 +
-                                                        16 * ks);
-      if (edge) {  // tokens past the last one may hold anything: a zero weight must not meet them
+      if (32 * b + 31 > p) {  // tokens past the last one may hold anything: a zero weight must not meet them
 #pragma unroll
         for (int i = 0; i < CW; ++i)
 #pragma unroll
           for (int ks = 0; ks < 2; ++ks)
 #pragma unroll
             for (int e = 0; e < 8; ++e)
-              if (32 * b + 16 * ks + 8 * (e >> 2) + 4 * hh + (e & 3) > p) vop[i][ks][e] = (__bf16)0.0f;
+              if (32 * b + 16 * ks + 8 * (e >> 2) + 4 * hh + (e & 3) > p) vop[w][i][ks][e] = (__bf16)0.0f;
       }
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
         const bf16x8 p1 = s_p[((w * 2 + ks) * 2 + 0) * 64 + lane], p2 = s_p[((w * 2 + ks) * 2 + 1) * 64 + lane];
 #pragma unroll
-        for (int i = 0; i < CW; ++i) acc[i] = mfma_bf16(vop[i][ks], p2, acc[i]);
+        for (int i = 0; i < CW; ++i) acc[i] = mfma_bf16(vop[w][i][ks], p2, acc[i]);
 #pragma unroll
-        for (int i = 0; i < CW; ++i) acc[i] = mfma_bf16(vop[i][ks], p1, acc[i]);
+        for (int i = 0; i < CW; ++i) acc[i] = mfma_bf16(vop[w][i][ks], p1, acc[i]);
       }
+    }
+    if (bt + kDecWaves < b_hi) {
+      load_k(bt + kDecWaves);
+      if (kAhead) load_v(bt + kDecWaves);
     }
     // the next tile's weights are written behind its first barrier, which is behind this tile's last read
   }
@@ -620,7 +681,7 @@ hipError_t rows_t(const LatentGeom& g, void* k, void* vt, const float* raw, void
                    g.eps, g.q_norm, g.kv_norm, g.sin_t, g.cos_t};
   const int lead = pos0 & (kRowTok - 1);
   const size_t lds = sizeof(float) * kRowTok * (g.kv_rank + g.rot_part);
-  hipLaunchKernelGGL(latent_rows_kernel<T>, dim3((M + lead + kRowTok - 1) / kRowTok), dim3(256), lds, s, raw,
+  hipLaunchKernelGGL(latent_rows_kernel<T>, dim3((M + lead + kRowTok - 1) / kRowTok), dim3(64 * kRowTok), lds, s, raw,
                      static_cast<T*>(cq), static_cast<T*>(k), static_cast<T*>(vt), M, pos0, a);
   return hipGetLastError();
 }
@@ -639,7 +700,7 @@ hipError_t absorb_t(const LatentGeom& g, void* k, void* vt, const float* raw, co
 template <int CW>
 hipError_t decode_cw(const LatentGeom& g, const void* k, const void* vt, const float* qa, const int* pos, int max_seq,
                      float* o, float* ml, hipStream_t s) {
-  const size_t lds = (size_t)(((g.Dc + g.Dr) / 16 + 7) / 8 * 8) * 1024 + kDecWaves * 4 * 1024 + sizeof(float) * 3 * kDecWaves * 32;
+  constexpr size_t lds = (size_t)8 * (CW + 1) * 1024 + kDecWaves * 4 * 1024 + sizeof(float) * 3 * kDecWaves * 32;
   auto kern = latent_decode_kernel<CW>;
   static LdsLimitOnce raised;
   if (hipError_t e = raised.raise(reinterpret_cast<const void*>(kern), 80 * 1024); e != hipSuccess) return e;

@@ -93,7 +93,6 @@ struct Geom {
 w4::MoeGeom moe_geom(const w4a32_layered_config* c, const w4a32_layer_config& l) {
   return {c->hidden, pad64(c->hidden), l.ff, pad64(l.ff), l.experts, l.top, l.expert_limit};
 }
-constexpr int kRouterParts = 8;  // most parts a router product is dealt to
 
 int check_config(const w4a32_layered_config* c) {
   if (!c || !c->layers) return W4A32_EINVAL;
@@ -315,7 +314,7 @@ Geom geometry(const w4a32_layered_config* c) {
   g.ve = take(g.elem * expand);
   g.qa = take(sizeof(float) * qa);
   g.head_out = take(sizeof(float) * head_out);
-  g.router = take(sizeof(float) * kRouterParts * Mb * pad64(experts));
+  g.router = take(sizeof(float) * w4::kMoeLogitParts * Mb * pad64(experts));
   g.moe = take(moe);
   g.sel = take(sizeof(int) * W4A32_LAYERED_MAX_TOP);
   g.ws_bytes = o;
@@ -488,7 +487,7 @@ int prefill_layers(const Run& r, const int64_t* tokens, int M, int pos0, int n_l
       W4_TRY(norm(lw.norm2, lw.canon2, g.st[i].canon2));
       int rp = 1;  // few tiles: dealt over k as far as that goes
       if (r.bf16()) {
-        rp = std::max(1, std::min(kRouterParts, Hp / 128));
+        rp = std::max(1, std::min(w4::kMoeLogitParts, Hp / 128));
         W4_LAUNCH(w4::launch_matmul_bf16(r.ws + g.y, lw.router, r.f32(g.router), M, Ep, Hp, Ep, false, rp, r.s));
       } else {
         W4_TRY(product(r, r.ws + g.y, lw.router, r.f32(g.router), M, Ep, Hp, false, nullptr));

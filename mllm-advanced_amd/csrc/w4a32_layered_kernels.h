@@ -222,6 +222,7 @@ struct MoeGeom {
   int hidden, Hp, ff, Fp, experts, top;
   float limit;
 };
+constexpr int kMoeLogitParts = 8;  // most of them
 size_t moe_scratch_bytes(int dtype, int M, int experts, int top, int Fp);
 // rows: h T [M][Hp], router logits f32 [logit_parts][M][ldl] -> parts f32 [top][M][Hp]
 hipError_t launch_moe_prefill(int dtype, const MoeGeom& g, const void* h, const float* logits, int logit_parts, int ldl,

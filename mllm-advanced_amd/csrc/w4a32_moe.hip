@@ -18,6 +18,7 @@ namespace w4 {
 namespace {
 
 constexpr float kGluAlpha = 1.702f;
+constexpr int kMaxParts = kMoeLogitParts;
 constexpr int kLogitRegs = W4A32_LAYERED_MAX_EXPERTS / 64;
 static_assert(W4A32_LAYERED_MAX_TOP <= 64, "a lane per chosen expert");
 
@@ -80,8 +81,11 @@ __global__ __launch_bounds__(256) void moe_choose_kernel(const float* __restrict
     v[i] = -INFINITY;
     if (e < experts) {
       const float* src = logits + (size_t)m * ldl + e;
-      float s = src[0];
-      for (int p = 1; p < parts; ++p) s += src[p * part_stride];
+      float x[kMaxParts], s = 0.0f;
+#pragma unroll
+      for (int p = 0; p < kMaxParts; ++p) x[p] = src[min(p, parts - 1) * part_stride];  // all requested before the first is used
+#pragma unroll
+      for (int p = 0; p < kMaxParts; ++p) s += p < parts ? x[p] : 0.0f;
       v[i] = s;
     }
   }
@@ -134,12 +138,21 @@ __global__ __launch_bounds__(kPlanThreads) void moe_plan_kernel(const int* __res
   const int e = blockIdx.x, tid = threadIdx.x;
   for (int i = tid; i < experts; i += kPlanThreads) s_count[i] = 0;
   __syncthreads();
+  // a thread takes a run of pairs, up to eight of them in registers
+  constexpr int kRegs = 8;
   const int per = (n + kPlanThreads - 1) / kPlanThreads, lo = min(n, tid * per), hi = min(n, lo + per);
-  int mine = 0;
-  for (int i = lo; i < hi; ++i) {
-    const int id = ids[i];
-    atomicAdd(&s_count[id], 1);
-    mine += id == e;
+  int mine = 0, id[kRegs];
+#pragma unroll
+  for (int i = 0; i < kRegs; ++i) id[i] = ids[min(lo + i, n - 1)];
+#pragma unroll
+  for (int i = 0; i < kRegs; ++i)
+    if (lo + i < hi) {
+      atomicAdd(&s_count[id[i]], 1);
+      mine += id[i] == e;
+    }
+  for (int i = lo + kRegs; i < hi; ++i) {
+    atomicAdd(&s_count[ids[i]], 1);
+    mine += ids[i] == e;
   }
   __syncthreads();
   int total;
@@ -149,7 +162,10 @@ __global__ __launch_bounds__(kPlanThreads) void moe_plan_kernel(const int* __res
   block_scan(before ? (s_count[tid] + bm - 1) / bm : 0, s_w, &total);
   const int first = total;
   int at = offset + block_scan(mine, s_w, &total);
-  for (int i = lo; i < hi; ++i)
+#pragma unroll
+  for (int i = 0; i < kRegs; ++i)
+    if (lo + i < hi && id[i] == e) order[at++] = lo + i;
+  for (int i = lo + kRegs; i < hi; ++i)
     if (ids[i] == e) order[at++] = i;
   const int count = total, mt = (count + bm - 1) / bm;
   for (int t = tid; t < mt; t += kPlanThreads)
@@ -374,6 +390,7 @@ hipError_t grouped(const MoeGeom& g, const T* h, const T* gate_up, const T* down
 template <typename T>
 hipError_t prefill_t(int dtype, const MoeGeom& g, const T* h, const float* logits, int logit_parts, int ldl, const T* gate_up,
                      const T* down, int M, float* parts, uint8_t* ws, hipStream_t s) {
+  if (logit_parts < 1 || logit_parts > kMaxParts) return hipErrorInvalidValue;
   const Scratch c = scratch_of(dtype, M, g.experts, g.top, g.Fp);
   const int bm = tile_rows(M, g.experts, g.top);
   int* ids = reinterpret_cast<int*>(ws + c.ids);

@@ -63,23 +63,31 @@ __global__ __launch_bounds__(256) void attn_qkv_kernel(const float* __restrict__
   const int head = cc / hd, d = cc - head * hd;
   T* dst = kind == 0 ? q + (size_t)head * D + d : (kind == 1 ? kc : vt) + (size_t)head * cap * D;
   const bool turn = ROT && kind < 2 && d < rot, store_v = kind == 2 || (ROT && tied && kind == 1);
-  const int partner = turn ? c + rot_partner(d, rot) - d : c;
+  const int partner = turn ? c + rot_partner(d, rot) - d : c, angle = turn ? (d < rot / 2 ? d : d - rot / 2) : 0;
   T* dst_v = vt + (size_t)head * cap * D;
   for (int tb = t0; tb < te;) {
     // up to the next multiple of eight positions
     const int n = min(te - tb, kQkvTok - ((pos0 + tb) & (kQkvTok - 1)));
     T out[kQkvTok], turned[kQkvTok];  // as projected (and convolved), and rotated
+    if constexpr (ROT) {
+      float x[kQkvTok], y[kQkvTok], sn[kQkvTok], cs[kQkvTok];
+#pragma unroll
+      for (int i = 0; i < kQkvTok; ++i) {  // all requested before the first is used
+        const int t = tb + min(i, n - 1);
+        x[i] = raw[(size_t)t * ldr + c];
+        y[i] = raw[(size_t)t * ldr + partner];
+        sn[i] = turn ? sin_t[(size_t)(pos0 + t) * (rot / 2) + angle] : 0.0f;
+        cs[i] = turn ? cos_t[(size_t)(pos0 + t) * (rot / 2) + angle] : 1.0f;
+      }
+#pragma unroll
+      for (int i = 0; i < kQkvTok; ++i) {
+        out[i] = (T)x[i];
+        turned[i] = (T)(partner > c ? x[i] * cs[i] - y[i] * sn[i] : x[i] * cs[i] + y[i] * sn[i]);
+      }
+    }
 #pragma unroll
     for (int i = 0; i < kQkvTok; ++i) {
-      if (i >= n) break;
-      if constexpr (ROT) {
-        const float x = raw[(size_t)(tb + i) * ldr + c];
-        out[i] = (T)x;
-        turned[i] = turn ? (T)rotated(x, raw[(size_t)(tb + i) * ldr + partner], d, rot, (size_t)(pos0 + tb + i), sin_t,
-                                      cos_t)
-                         : out[i];
-        continue;
-      }
+      if (ROT || i >= n) break;
       win[0] = raw[(size_t)(tb + i) * ldr + c];
       float acc = 0.0f;
 #pragma unroll
@@ -520,6 +528,19 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
   constexpr int kAhead = 2, kFastTaps = 4;
   const bool ahead = taps > 0 && taps <= kFastTaps;
   float cx[kAhead], cw[kAhead][kFastTaps], cr[kAhead][kFastTaps];
+  if (taps == 0) {  // a rotated channel's partner and angle instead
+#pragma unroll
+    for (int i = 0; i < kAhead; ++i) {
+      const int it = tid + kDecThreads * i, r = it / D, d = it - r * D, c = max(channel(it), 0);
+      const bool turn = d < rot && r <= rep && it < items;
+      const int a = turn ? (d < rot / 2 ? d : d - rot / 2) : 0;
+      cx[i] = raw[c];
+      cr[i][0] = turn ? raw[c + rot_partner(d, rot) - d] : 0.0f;
+      cw[i][0] = turn ? cos_t[(size_t)p * (rot / 2) + a] : 1.0f;
+      cw[i][1] = turn ? sin_t[(size_t)p * (rot / 2) + a] : 0.0f;
+      if (d < rot / 2) cw[i][1] = -cw[i][1];
+    }
+  }
   if (ahead) {
 #pragma unroll
     for (int i = 0; i < kAhead; ++i) {
@@ -554,7 +575,6 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
     if (c >= 0) {
       const int r = it / D, d = it - r * D;
       if (taps > 0 && slice == 0) ring[(size_t)(p % taps) * ldc + c] = x;
-      if (d < rot && r <= rep) y = rotated(x, raw[c + rot_partner(d, rot) - d], d, rot, (size_t)p, sin_t, cos_t);
       y = (float)(T)y;
       if (slice == 0) {
         if (r == rep) kb[k_at(p, d, D)] = (T)y;
@@ -575,10 +595,20 @@ __global__ __launch_bounds__(kDecThreads) void attn_decode_kernel(
       if (it < items) finish(it, channel(it), cx[i], __fmaf_rn(cw[i][0], cx[i], y));
     }
   }
-  for (int it = tid + (ahead ? kAhead * kDecThreads : 0); it < items; it += kDecThreads) {
-    const int c = channel(it);
+  if (taps == 0) {
+#pragma unroll
+    for (int i = 0; i < kAhead; ++i) {
+      const int it = tid + kDecThreads * i;
+      if (it < items) finish(it, channel(it), cx[i], cx[i] * cw[i][0] + cr[i][0] * cw[i][1]);
+    }
+  }
+  for (int it = tid + (ahead || taps == 0 ? kAhead * kDecThreads : 0); it < items; it += kDecThreads) {
+    const int c = channel(it), r = it / D, d = it - r * D;
     const float x = raw[max(c, 0)];
-    finish(it, c, x, taps > 0 ? conv_step(x, conv, ring, max(c, 0), ldc, taps, p) : x);
+    const bool turn = c >= 0 && d < rot && r <= rep;
+    finish(it, c, x,
+           turn ? rotated(x, raw[c + rot_partner(d, rot) - d], d, rot, (size_t)p, sin_t, cos_t)
+                : taps > 0 ? conv_step(x, conv, ring, max(c, 0), ldc, taps, p) : x);
   }
   for (int it = tid; it < rep * D; it += kDecThreads) s_o[it] = 0.0f;
   for (int r = tid; r < rep; r += kDecThreads) {
