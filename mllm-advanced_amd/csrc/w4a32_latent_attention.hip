@@ -79,18 +79,22 @@ template <typename T>
 __global__ __launch_bounds__(64 * kRowTok) void latent_rows_kernel(const float* __restrict__ raw, T* __restrict__ cq,
                                                                    T* __restrict__ kc, T* __restrict__ vt, int M, int pos0,
                                                                    const RowsArgs a) {
-  extern __shared__ __align__(16) float s_c[];  // [kRowTok][kv_rank + rot_part]
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, ld = a.kv_rank + a.rot_part;
+  extern __shared__ __align__(16) float s_c[];  // [kRowTok][ld], ld odd: the eight tokens' rows start on other banks
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, ld = (a.kv_rank + a.rot_part) | 1;
   const int lead = pos0 & (kRowTok - 1);
   const int t0 = max(0, (int)blockIdx.x * kRowTok - lead), te = min(M, ((int)blockIdx.x + 1) * kRowTok - lead);
   const int t = t0 + wave;
   if (t < te) {
     const float* row = raw + (size_t)t * a.ldr;
     constexpr int kRegs = 16;  // a query latent of up to 1024 stays in registers
-    float x[kRegs], ss = 0.0f;
+    float x[kRegs], w[kRegs], ss = 0.0f;
     if (a.ldq <= 64 * kRegs) {
 #pragma unroll
-      for (int i = 0; i < kRegs; ++i) x[i] = row[min(lane + 64 * i, a.q_rank - 1)];
+      for (int i = 0; i < kRegs; ++i) {
+        const int d = min(lane + 64 * i, a.q_rank - 1);
+        x[i] = 64 * i < a.q_rank ? row[d] : 0.0f;
+        w[i] = 64 * i < a.q_rank ? a.q_norm[d] : 0.0f;
+      }
       latent_of_row(row, a.kv_rank, a.rot_part, a.rot_dims, a.kv_off, a.rot_off, a.kv_norm, a.eps, pos0 + t, a.sin_t,
                     a.cos_t, s_c + (size_t)wave * ld);
 #pragma unroll
@@ -102,7 +106,7 @@ __global__ __launch_bounds__(64 * kRowTok) void latent_rows_kernel(const float* 
 #pragma unroll
       for (int i = 0; i < kRegs; ++i) {
         const int d = lane + 64 * i;
-        if (d < a.ldq) cq[(size_t)t * a.ldq + d] = (T)(x[i] * r * a.q_norm[d]);
+        if (d < a.ldq) cq[(size_t)t * a.ldq + d] = (T)(x[i] * r * w[i]);
       }
     } else {
       latent_of_row(row, a.kv_rank, a.rot_part, a.rot_dims, a.kv_off, a.rot_off, a.kv_norm, a.eps, pos0 + t, a.sin_t,
@@ -680,7 +684,7 @@ hipError_t rows_t(const LatentGeom& g, void* k, void* vt, const float* raw, void
   const RowsArgs a{g.q_rank, g.kv_rank, g.rot_part, g.rot_dims, g.Dc, g.Dr, g.ldr, g.kv_off, g.rot_off, ldq,
                    g.eps, g.q_norm, g.kv_norm, g.sin_t, g.cos_t};
   const int lead = pos0 & (kRowTok - 1);
-  const size_t lds = sizeof(float) * kRowTok * (g.kv_rank + g.rot_part);
+  const size_t lds = sizeof(float) * kRowTok * ((g.kv_rank + g.rot_part) | 1);
   hipLaunchKernelGGL(latent_rows_kernel<T>, dim3((M + lead + kRowTok - 1) / kRowTok), dim3(64 * kRowTok), lds, s, raw,
                      static_cast<T*>(cq), static_cast<T*>(k), static_cast<T*>(vt), M, pos0, a);
   return hipGetLastError();

@@ -76,6 +76,58 @@ def test_rotation_is_relative_and_leaves_the_rest():
                        [u * np.cos(2) - v * np.sin(2), v * np.cos(2) + u * np.sin(2)])
 
 
+def test_sink_attention_against_torch_with_one_more_key():
+    """A sink is a key whose score is the sink and whose value is zero."""
+    T, H, G, d, dv = 17, 4, 2, 8, 6
+    q, k, v = rng.standard_normal((T, H, d)), rng.standard_normal((T, G, d)), rng.standard_normal((T, G, dv))
+    sinks = rng.standard_normal(H) * 2
+    for size in (None, 1, 5, 40):
+        i, j = np.arange(T)[:, None], np.arange(T)[None]
+        mask = np.where((j <= i) & (i - j < (size or T)), 0.0, -np.inf)
+        mask = np.concatenate([np.repeat(mask[None], H, 0), np.repeat(sinks[:, None, None], T, 1)], 2)
+        more = lambda x: torch.tensor(np.concatenate([np.repeat(x, 2, 1).transpose(1, 0, 2), np.zeros((H, 1, x.shape[2]))], 1))
+        ref = torch.nn.functional.scaled_dot_product_attention(torch.tensor(q.transpose(1, 0, 2)), more(k), more(v),
+                                                               attn_mask=torch.tensor(mask), scale=0.4).numpy()
+        assert np.allclose(lo.sink_attention(q, k, v, 0.4, sinks, size), ref.transpose(1, 0, 2))
+
+
+def test_latent_attention_reads_what_its_folded_form_reads():
+    """Scores and values taken in the latent space: query times W_uk, output times W_uv."""
+    cfg = lm.lesarax([lm.latent(3, 6, 4, 5, 9, 7, 4)], width=12)
+    w, m = lm.lesarax_weights(cfg, seed=2), cfg["layers"][0]["mixer"]
+    p, T, H = "l0.mix.", 11, 3
+    h = rng.standard_normal((T, 12))
+    q = (lo.rms_norm(h @ w[p + "dq"].T, w[p + "dq.norm"], 1e-5) @ w[p + "uq"].T).reshape(T, H, 10)
+    ckv = h @ w[p + "dkv"].T
+    c, uk, uv = lo.rms_norm(ckv[:, :7], w[p + "dkv.norm"], 1e-5), w[p + "uk"].reshape(3, 6, 7), w[p + "uv"].reshape(3, 5, 7)
+    out = np.zeros((T, H, 5))
+    for t in range(T):
+        seen = range(max(0, t - 3), t + 1)
+        for i in range(H):
+            qr = lo.rotate_half(q[t, i, 6:], t, 4, 3000.0)
+            s = [(uk[i].T @ q[t, i, :6]) @ c[j] + qr @ lo.rotate_half(ckv[j, 7:], j, 4, 3000.0) for j in seen]
+            e = np.exp(np.array(s) * m["scale"])
+            out[t, i] = uv[i] @ (e @ c[list(seen)]) / (e.sum() + np.exp(w[p + "sink"][i]))
+            out[t, i] *= lo.sigmoid(w[p + "g"] @ h[t])[i]
+    assert np.allclose(lo.mixer_latent_attention(cfg, w, p, m, h), out.reshape(T, -1) @ w[p + "o"].T)
+
+
+def test_experts_norm_and_layer_runs():
+    x = rng.standard_normal((4, 9))
+    assert np.allclose(lo.rms_norm(x, np.ones(9), 0.0), torch.nn.functional.rms_norm(torch.tensor(x), (9,)).numpy())
+    pick, a = lo.route(np.array([0.1, 3.0, -2.0, 2.0]), 2)
+    assert list(pick) == [1, 3] and np.allclose(a, [1 / (1 + np.exp(-1)), 1 / (1 + np.exp(1))])
+    one, zero = np.eye(3), np.zeros((3, 3))
+    h = np.array([0.5, -0.7, 4.0])
+    g = np.minimum(h, 1.5)
+    assert np.allclose(lo.clamped_expert(h, one, zero, one, 1.5), g * lo.sigmoid(1.702 * g))
+    assert np.allclose(lo.clamped_expert(h, one, one, 2 * one, 1.5), 2 * g * lo.sigmoid(1.702 * g) * (np.clip(h, -1.5, 1.5) + 1))
+    assert np.allclose(lo.clamped_expert(-h, one, one, one, 1.5)[2], -4 * lo.sigmoid(1.702 * -4.0) * -0.5)   # g has no lower limit
+    layers = [lm.rotary(1, 1, 8, 4)] * 4
+    assert lo.layer_runs(lm.lesarax(layers, loop=(1, 3, 2))) == [(0, 0), (1, 1), (2, 0), (1, 1), (2, 0), (3, 0)]
+    assert lo.layer_runs(lm.lesarax(layers, loop=(0, 1, 3))) == [(0, 1), (0, 1), (0, 1), (1, 0), (2, 0), (3, 0)]
+
+
 def test_safetensors_round_trip(tmp_path):
     w = {"a.b": lo.bf16_round(rng.standard_normal((3, 5))), "c": lo.bf16_round(rng.standard_normal(7) * 1e-3)}
     lo.save_safetensors(tmp_path / "m", w)
@@ -131,6 +183,57 @@ def test_configurations_that_cannot_run_are_refused(pkg):
     assert code([R], field(0, "mixer", 9)) == EINVAL
     assert code([A], taps=0) == EINVAL and code([A], taps=9) == ENOTSUP
     assert code([A], lambda cfg, arr: setattr(cfg, "dtype", 3)) == EINVAL
+
+
+def test_rotary_latent_experts_and_loops_are_checked(pkg):
+    L = pkg.lib()
+
+    def cfg_of(change=None, experts=4, loop=(0, 1, 2)):
+        arr = (pkg.LayerConfig * 2)()
+        a, b = arr
+        a.mixer, a.heads, a.kv_heads, a.dim, a.vdim, a.kv_from = pkg.MIXERS["rotary"], 4, 2, 24, 24, -1
+        a.tied_values, a.rot_dims, a.rot_base, a.scale = 1, 12, 1e4, 0.2
+        b.mixer, b.heads, b.kv_heads, b.dim, b.vdim, b.kv_from = pkg.MIXERS["latent"], 3, 3, 24, 20, -1
+        b.q_rank, b.kv_rank, b.rot_part, b.rot_dims, b.rot_base, b.scale, b.window = 30, 40, 8, 8, 1e4, 0.2, 5
+        for c in arr:
+            c.ff, c.experts, c.top, c.expert_limit = 32, experts, 2, 1.0
+        cfg = pkg.LayeredConfig(48, 30, 2, 0, 1e-5, 1, 64, 16, arr, pkg.NORM_RMS, 0.5, *loop)
+        if change:
+            change(cfg, a, b)
+        return cfg, arr
+
+    def code(change=None, **kw):
+        cfg, arr = cfg_of(change, **kw)
+        return L.w4a32_layered_check(ctypes.byref(cfg))
+
+    def set_(i, **kw):
+        return lambda *c: [setattr(c[i], k, v) for k, v in kw.items()]
+
+    EINVAL, ESHAPE, ENOTSUP = -1, -2, -4
+    assert code() == 0
+    assert code(set_(0, norm=pkg.NORM_LAYER)) == EINVAL        # layer norm comes with the input convolution
+    assert code(set_(0, norm=7)) == EINVAL
+    assert code(set_(0, loop_times=-1)) == EINVAL
+    assert code(loop=(1, 3, 2)) == ESHAPE and code(loop=(1, 1, 2)) == ESHAPE and code(loop=(-1, 1, 2)) == ESHAPE
+    assert code(loop=(0, 0, 0)) == 0
+    assert code(set_(1, rot_dims=13)) == ESHAPE and code(set_(1, rot_dims=26)) == ESHAPE
+    assert code(set_(1, vdim=20)) == ESHAPE                     # tied values are as long as the keys
+    assert code(set_(1, vdim=20, tied_values=0)) == 0
+    assert code(set_(1, conv_taps=3)) == ENOTSUP and code(set_(1, heads=66)) == ENOTSUP
+    assert code(set_(1, rot_base=0.0)) == EINVAL and code(set_(1, window=-1)) == EINVAL
+    assert code(set_(2, kv_heads=1)) == ESHAPE and code(set_(2, rot_dims=10)) == ESHAPE
+    assert code(set_(2, q_rank=0)) == EINVAL and code(set_(2, kv_rank=0)) == EINVAL
+    assert code(set_(2, kv_rank=513)) == ENOTSUP and code(set_(2, rot_part=130)) == ENOTSUP
+    assert code(set_(2, window=0)) == 0 and code(set_(2, rot_part=0, rot_dims=0)) == 0
+    assert code(set_(1, top=5)) == EINVAL and code(set_(1, top=0)) == EINVAL and code(set_(1, expert_limit=0.0)) == EINVAL
+    assert code(experts=513) == ENOTSUP and code(set_(1, experts=64, top=17)) == ENOTSUP
+    assert code(set_(1, ff=40000)) == ENOTSUP
+    # a looped layer has a cache per pass; a latent layer keeps its latent and key part only
+    runs = lambda **kw: (lambda c: (L.w4a32_layered_runs(ctypes.byref(c[0])), L.w4a32_layered_state_bytes(ctypes.byref(c[0]))))(
+        cfg_of(**kw))
+    (n1, one), (n3, three) = runs(loop=(0, 1, 1)), runs(loop=(0, 1, 3))
+    assert (n1, n3) == (2, 4) and three - one == 2 * 2 * 2 * 2 * 64 * 32
+    assert L.w4a32_layered_head_rows(24, 20) == 32 and L.w4a32_layered_head_rows(24, 130) == 256
 
 
 def test_a_layer_that_reads_another_ones_keys_keeps_no_cache_of_its_own(pkg):
