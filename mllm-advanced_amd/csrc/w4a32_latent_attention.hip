@@ -86,7 +86,7 @@ __global__ __launch_bounds__(64 * kRowTok) void latent_rows_kernel(const float* 
   const int t = t0 + wave;
   if (t < te) {
     const float* row = raw + (size_t)t * a.ldr;
-    constexpr int kRegs = 16;  // a query latent of up to 1024 stays in registers
+    constexpr int kRegs = 32;  // a query latent of up to 2048 stays in registers
     float x[kRegs], w[kRegs], ss = 0.0f;
     if (a.ldq <= 64 * kRegs) {
 #pragma unroll
