@@ -31,6 +31,7 @@ def test_flags_and_algorithmic_bytes():
     finally:
         sys.argv = argv
     assert args.gpus == 1 and args.steps > 0 and args.warmup >= 0
+    assert args.layered is None and args.lesarax is None             # other workloads are asked for
 
 
 def test_traffic_constant_is_the_one_the_counter_profile_derives():
